@@ -210,7 +210,9 @@ class MixerSpec:
     are its keys, without positions) | "time_mix" (linear attention with a
     learned decay per key channel and a bonus for the current token, on inputs
     mixed with the previous token's) | "parallel" (two mixers side by side on
-    the same input, their scaled outputs summed)."""
+    the same input, their scaled outputs summed) | "gated_rotary" (rotary
+    softmax attention with a window, kept first tokens, values mixed with an
+    earlier layer's and an output gate per channel)."""
 
     kind: str
     heads: int
@@ -224,14 +226,29 @@ class MixerSpec:
     decay_rank: Optional[int] = None
     gate_rank: Optional[int] = None
     # rotary attention: rotated channels per head (0 = none), frequency base,
-    # wavelength-dependent rescaling {factor, low, high, original} or None
+    # rescaling by wavelength {factor, low, high, original} or by pair index
+    # {factor, fast, slow, original} (see rotary_inv_freq), or None
     rot_dims: int = 0
     rot_base: float = 10000.0
     rot_scaling: Optional[dict] = None
     # keys a query sees, itself included (None = all earlier keys)
     window: Optional[int] = None
+    # keys at positions below keep_first are seen from beyond the window too
+    keep_first: int = 0
     # a learned per-head term in the softmax denominator
     sink: bool = False
+    # a sink of fixed score 0: one is added to the softmax denominator
+    plus_one: bool = False
+    # per-head RMS norm of queries and keys: "weighted" (before the rotation,
+    # a weight per channel) or "unit_rotated" (after it, no weight)
+    qk_norm: str = "weighted"
+    # biases on the query, key and value projections
+    qkv_bias: bool = False
+    # values are mixed with those of the first layer that has v_mix:
+    # v <- (1 - lambda) v + lambda v_first. v_first_from names that layer
+    # (None: this is it, or no mixing)
+    v_mix: bool = False
+    v_first_from: Optional[int] = None
     # latent attention: size of the cached latent, rotated channels per head
     # (query) and of the shared key part, and the layer whose cached latent
     # this layer reads instead of projecting its own (None = its own)
@@ -266,7 +283,8 @@ class MixerSpec:
     def has_kv(self) -> bool:
         if self.kind == "parallel":
             return self.left.has_kv or self.right.has_kv
-        return self.kind in ("attention", "rotary_window", "diff_attention", "key_attention") or (
+        return self.kind in ("attention", "rotary_window", "diff_attention", "key_attention",
+                             "gated_rotary") or (
             self.kind == "latent_attention" and self.kv_from is None)
 
     @property
@@ -342,8 +360,12 @@ class HybridSpec:
     # "hyper": pre-norm sublayers (layer norm with weight and bias) around
     # `streams` residual streams joined by learned hyper-connections.
     # "parallel": one dynamic-tanh norm per layer, mixer and feed-forward both
-    # read it and are added together.
+    # read it and are added together. "parallel_rms": the same with an RMS
+    # norm of its own for each sublayer (weights stored as distances from 1)
+    # and a gated feed-forward.
     layer_style: str = "post_canon"
+    # an RMS norm (weight stored as its distance from 1) follows the embedding
+    embed_norm: bool = False
     embed_scale: float = 1.0
     streams: int = 1
     # learned read/mix/write coefficients between the streams (False: the
@@ -937,12 +959,112 @@ def rimonex_config_dict(
     return cfg
 
 
+def rope_scaling_of(rot: dict) -> Optional[dict]:
+    """A config's rot.scaling as a plain dictionary of floats; None if absent."""
+    return {k: float(v) for k, v in rot["scaling"].items()} if rot.get("scaling") else None
+
+
+def safesun_spec_from_dict(cfg: dict, name: str = "safesun") -> HybridSpec:
+    """Parse a Safesun config.json dict: layers whose mixer and silu
+    feed-forward each read their own RMS norm of the same stream; two kinds of
+    gated rotary attention (weighted query/key norms before the rotation; or
+    biases, unit query/key after it and one added to the softmax denominator),
+    windows with kept first tokens, values mixed with the first value-mixing
+    layer's; a norm after the embedding; the head is the embedding table."""
+    layers, first = [], None
+    for i, entry in enumerate(cfg["layers"]):
+        kind, m = entry["type"], entry["mixer"]
+        if kind not in ("attention", "attention_2"):
+            raise ValueError(f"unknown Safesun layer type {kind!r}")
+        second = kind == "attention_2"
+        rot, mask = m.get("rot") or {}, m.get("mask") or {}
+        mixer = MixerSpec(
+            kind="gated_rotary", heads=int(m["heads"]), kv_heads=int(m["kv_heads"]),
+            dim=int(m["dim"]), vdim=int(m["vdim"]),
+            scale=float(m["scale"]) if "scale" in m else None,
+            rot_dims=int(rot.get("dims", 0)), rot_base=float(rot.get("base", 10000.0)),
+            rot_scaling=rope_scaling_of(rot), rot_layout="half",
+            window=int(mask["size"]) if mask.get("size") else None,
+            keep_first=int(mask.get("keep_first") or 0), plus_one=second, qkv_bias=second,
+            qk_norm="unit_rotated" if second else "weighted", v_mix=bool(m.get("v_mix")),
+            gate="channel",
+        )
+        if mixer.heads % mixer.kv_heads:
+            raise ValueError("heads must be a multiple of kv_heads")
+        if mixer.rot_dims % 2 or mixer.rot_dims > mixer.dim:
+            raise ValueError("rot.dims must be even and at most dim")
+        if mixer.v_mix:
+            if first is None:
+                first = i
+            else:
+                o = layers[first].mixer
+                if (o.kv_heads, o.vdim) != (mixer.kv_heads, mixer.vdim):
+                    raise ValueError(f"layer {i}: mixed values need layer {first}'s kv_heads and vdim")
+                mixer.v_first_from = first
+        mlp = entry.get("mlp")
+        ls = HybridLayerSpec(mixer=mixer)
+        if mlp is not None:
+            if mlp.get("kind", "dense") != "dense":
+                raise ValueError(f"unknown Safesun feed-forward kind {mlp.get('kind')!r}")
+            ls.mlp_kind, ls.mlp_ff, ls.mlp_act = "dense", int(mlp["ff"]), "silu"
+        layers.append(ls)
+    return HybridSpec(
+        name=name, architecture="Safesun", vocab_size=int(cfg["vocab"]),
+        hidden_size=int(cfg["width"]), layers=layers, norm_eps=float(cfg["norm"]["eps"]),
+        layer_style="parallel_rms", embed_norm=True, tied_head=True,
+    )
+
+
+def safesun_config_dict(
+    vocab: int, width: int, pattern: str, heads: int = 4, kv_heads: int = 2, dim: int = 16,
+    vdim: int = 16, window: Optional[int] = 24, keep_first: int = 4, scale: Optional[float] = None,
+    rot_dims: Optional[int] = None, rot_base: float = 10000.0, rot_scaling: Optional[dict] = None,
+    heads_2: Optional[int] = None, dim_2: Optional[int] = None, window_2: Optional[int] = None,
+    keep_first_2: Optional[int] = None, scale_2: Optional[float] = None,
+    rot_dims_2: Optional[int] = None, rot_base_2: float = 500000.0, ff: int = 128,
+    eps: float = 1e-5,
+) -> dict:
+    """A Safesun config.json dict from a layer pattern, two characters per
+    layer: the mixer 'A' (attention) or 'B' (attention_2), lower case without
+    value mixing, then the feed-forward 'd' (dense) or '-' (none). Parameters
+    with _2 are attention_2's (default: attention's)."""
+    if len(pattern) % 2:
+        raise ValueError("pattern: two characters per layer")
+    layers = []
+    for i in range(0, len(pattern), 2):
+        mk, fk = pattern[i], pattern[i + 1]
+        if mk not in "AaBb":
+            raise ValueError(f"unknown mixer letter {mk!r}")
+        if fk not in "d-":
+            raise ValueError(f"unknown feed-forward letter {fk!r}")
+        if mk in "Aa":
+            h, d, win, keep, sc = heads, dim, window, keep_first, scale
+            rot = {"base": rot_base, "dims": d if rot_dims is None else rot_dims}
+            if rot_scaling:
+                rot["scaling"] = dict(rot_scaling)
+        else:
+            h, d = heads_2 or heads, dim_2 or dim
+            win = window if window_2 is None else window_2
+            keep = keep_first if keep_first_2 is None else keep_first_2
+            sc = scale_2
+            rot = {"base": rot_base_2, "dims": d if rot_dims_2 is None else rot_dims_2}
+        mixer = {"heads": h, "kv_heads": kv_heads, "dim": d, "vdim": vdim, "rot": rot,
+                 "scale": sc if sc is not None else d ** -0.5, "v_mix": mk.isupper()}
+        if win:
+            mixer["mask"] = {"size": win, "keep_first": keep}
+        layers.append({"type": "attention" if mk in "Aa" else "attention_2", "mixer": mixer,
+                       "mlp": {"kind": "dense", "ff": ff} if fk == "d" else None})
+    return {"architecture": "Safesun", "layers": layers, "norm": {"eps": eps}, "vocab": vocab,
+            "width": width}
+
+
 # config.json "architecture" -> parser
 ARCHITECTURE_PARSERS = {"Povazen": povazen_spec_from_dict,
                         "Vazilorn": vazilorn_spec_from_dict,
                         "Rafodra": rafodra_spec_from_dict,
                         "Suzulix": suzulix_spec_from_dict,
-                        "Rimonex": rimonex_spec_from_dict}
+                        "Rimonex": rimonex_spec_from_dict,
+                        "Safesun": safesun_spec_from_dict}
 
 # named hybrid configurations (random-weight benchmarking and tests)
 HYBRID_REGISTRY = {
@@ -1039,6 +1161,24 @@ HYBRID_REGISTRY = {
     "rimonex-4l4k": lambda: rimonex_config_dict(
         vocab=2048, width=4096, pattern="PdDdPdDd", heads=32, kv_heads=8, dim=128, window=1024,
         mix_heads=32, mix_dim=128, delta_heads=32, delta_dim=128, delta_vdim=128, ff=14336),
+    # CPU-test size: both mixers with and without value mixing, a layer without feed-forward
+    "safesun-tiny": lambda: safesun_config_dict(
+        vocab=512, width=64, pattern="adBdA-Bd", heads=4, kv_heads=2, dim=16, vdim=24, window=24,
+        keep_first=3, rot_dims=12, window_2=20, keep_first_2=5, ff=96,
+        rot_scaling={"factor": 4.0, "fast": 16.0, "slow": 1.0, "original": 64}),
+    # GPU-smoke size
+    "safesun-micro": lambda: safesun_config_dict(
+        vocab=2048, width=1024, pattern="AdBdBdAd", heads=8, kv_heads=2, dim=128, vdim=128,
+        window=512, keep_first=4, rot_dims_2=64, ff=2816,
+        rot_scaling={"factor": 8.0, "fast": 32.0, "slow": 1.0, "original": 4096}),
+    # layer shapes of ~1B- and ~8B-class models at 4 layers (speed beside
+    # Vazilorn layers of equal width)
+    "safesun-4l2k": lambda: safesun_config_dict(
+        vocab=2048, width=2048, pattern="AdBdBdAd", heads=16, kv_heads=4, dim=128, vdim=128,
+        window=1024, keep_first=4, ff=8192),
+    "safesun-4l4k": lambda: safesun_config_dict(
+        vocab=2048, width=4096, pattern="AdBdBdAd", heads=32, kv_heads=8, dim=128, vdim=128,
+        window=1024, keep_first=4, ff=14336),
 }
 
 

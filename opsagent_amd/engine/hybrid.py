@@ -1,5 +1,5 @@
 """Hybrid decoders: a per-layer choice of token mixer and feed-forward
-around a float32 residual stream, in five layer styles.
+around a float32 residual stream, in six layer styles.
 
 "post_canon" (the Povazen design): softmax attention with a linear distance
 penalty, or a gated delta rule with per-channel decay.
@@ -42,6 +42,16 @@ projection of a layer is one weight, and so is every output projection.
 Sinusoidal positions at the embedding; a looped run of layers adds the
 embedding output again before every later pass. The head is the embedding
 table.
+
+"parallel_rms" (the Safesun design): rotary windowed attention that also keeps
+the first tokens in sight, in two kinds (weighted query/key norms before the
+rotation; or biases, unit queries and keys after it, and one added to the
+softmax denominator), values mixed with an earlier layer's, an output gate per
+channel; gated silu feed-forwards.
+Layer:  x <- x + (mixer(norm1(x)) + ff(norm2(x))), both RMS norms of the same
+x with weights stored as distances from one: the normed inputs are two planes
+of one launch, the projections as in "parallel". An RMS norm follows the
+embedding. The head is the embedding table.
 
 The mixers are modules of their own (BiasedAttentionMixer,
 ChannelDeltaMixer, ...) with every constant a constructor argument, built on the
@@ -628,9 +638,12 @@ class InputRows:
     sources: List[str]
     plane: int = 0
     act: Optional[str] = None
+    # the rows of two sources alternate (a_0, b_0, a_1, b_1, ...): what a
+    # gated activation needs side by side
+    paired: bool = False
 
 
-# Mixers of the "parallel" layer style own no projections: they name their
+# Mixers of the "parallel" layer styles own no projections: they name their
 # input rows, read the projected columns by key and write the columns of the
 # layer's one output projection.
 
@@ -733,6 +746,97 @@ class KeyAttentionMixer(nn.Module):
             put(self.sinks, [get(p + "sink")])
 
 
+class GatedRotaryMixer(nn.Module):
+    """Causal softmax attention with rotary positions, a window and an output
+    gate. Every option is a MixerSpec field:
+      qkv_bias     biases on the query, key and value projections;
+      qk_norm      queries and keys are divided by the root mean square of
+                   their head's channels: "weighted", before the rotation and
+                   times a weight per channel shared by the heads, or
+                   "unit_rotated", after the rotation and without a weight;
+      rot_*        rotated channels, base, rescaling of the frequencies (which
+                   may also scale the rotated channels, rotary_magnitude);
+      window, keep_first   position i sees j <= i if i - j < window or
+                   j < keep_first; kept tokens keep their true positions;
+      plus_one     the softmax denominator holds one more term, exp(0);
+      v_mix        v <- (1 - lambda) v + lambda v_first, v_first the same
+                   token's values in layer v_first_from. That layer's cache
+                   holds exactly those, at the slot the token has here too, so
+                   they are read from there; the mixed v is what is cached.
+    The heads' outputs times sigmoid(W_g h), element by element, are this
+    mixer's columns of the output projection."""
+
+    bias_source = None
+    out_scale = 1.0
+    mu_names: List[str] = []
+
+    def __init__(self, hidden: int, m: MixerSpec, eps: float, dtype, gen):
+        super().__init__()
+        self.H, self.G, self.D, self.Dv = m.heads, m.kv_heads, m.dim, m.vdim
+        self.eps = eps
+        self.scale = float(m.scale) if m.scale is not None else m.dim ** -0.5
+        self.window = int(m.window) if m.window else None
+        self.keep_first = int(m.keep_first)
+        self.layout, self.rot_dims = m.rot_layout, m.rot_dims
+        self.unit_rotated = m.qk_norm == "unit_rotated"
+        self.v_first_from = m.v_first_from
+        H, G, D, Dv, dev = self.H, self.G, self.D, self.Dv, gen.device
+        self.n_qkv = (H + G) * D + G * Dv
+        self.qkv_b = _param(_rand(gen, self.n_qkv, std=0.02, dtype=dtype)) if m.qkv_bias else None
+        self.q_norm_w = self.k_norm_w = None
+        if not self.unit_rotated:
+            self.q_norm_w = _param(1.0 + 0.1 * _rand(gen, D))
+            self.k_norm_w = _param(1.0 + 0.1 * _rand(gen, D))
+        self.lam = _param(torch.full((1,), 0.5, device=dev)) if m.v_first_from is not None else None
+        self.register_buffer("sinks", torch.zeros(H, device=dev) if m.plus_one else None,
+                             persistent=False)
+        self.register_buffer(
+            "inv_freq", mx.rotary_inv_freq(m.rot_dims, m.rot_base, m.rot_scaling).to(dev),
+            persistent=False)
+        self.magnitude = mx.rotary_magnitude(m.rot_scaling)
+        self.outputs = [("o", H * Dv)]
+
+    def inputs(self) -> List[InputRows]:
+        return [InputRows("qkv", self.n_qkv, ["q", "k", "v"]),
+                InputRows("g", self.H * self.Dv, ["g"])]
+
+    def kv_shape(self):
+        return (self.G, self.D, self.Dv)
+
+    def state_shapes(self) -> Dict[str, tuple]:
+        return {}
+
+    def forward(self, p, sb: mx.SeqBatch, kv, state, outs) -> None:
+        k_cache, v_cache = kv[:2]
+        first = kv[2] if self.lam is not None else None
+        q = mx.attn_rope_prepare(p["qkv"], self.q_norm_w, self.k_norm_w, self.inv_freq, self.H,
+                                 self.G, self.D, self.Dv, self.eps, k_cache, v_cache, sb,
+                                 bias=self.qkv_b, unit_rotated=self.unit_rotated,
+                                 magnitude=self.magnitude, v_first=first, v_lambda=self.lam)
+        mx.attention_paged(q, k_cache, v_cache, sb, self.scale, window=self.window,
+                           keep_first=self.keep_first, sinks=self.sinks, gate_logits=p["g"],
+                           gate_channels=True, out=outs["o"])
+
+    def load(self, get, put, p: str) -> None:
+        relay = lambda w, heads: _relayout_heads(w, heads, self.D, 0, self.rot_dims,  # noqa: E731
+                                                 self.layout).reshape(-1)
+        if self.qkv_b is not None:
+            put(self.qkv_b, [relay(get(p + "q.b"), self.H), relay(get(p + "k.b"), self.G),
+                             get(p + "v.b")])
+        if self.q_norm_w is not None:
+            put(self.q_norm_w, [relay(get(p + "q.norm"), 1)])
+            put(self.k_norm_w, [relay(get(p + "k.norm"), 1)])
+        if self.lam is not None:
+            put(self.lam, [get(p + "vmix")])
+
+    def source_rows(self, name: str, w: torch.Tensor) -> torch.Tensor:
+        """Input rows as the layer's weight holds them."""
+        if name not in ("q", "k"):
+            return w
+        return _relayout_heads(w, self.H if name == "q" else self.G, self.D, 0, self.rot_dims,
+                               self.layout)
+
+
 class TimeMixMixer(nn.Module):
     """Linear attention with a learned decay per head and key channel and a
     bonus for the current token. With h' the previous token's input each of
@@ -828,7 +932,8 @@ class SideBySideMixer(nn.Module):
 
 
 PART_MIXERS = {"head_delta": HeadDeltaMixer, "key_attention": KeyAttentionMixer,
-               "time_mix": TimeMixMixer, "parallel": SideBySideMixer}
+               "time_mix": TimeMixMixer, "parallel": SideBySideMixer,
+               "gated_rotary": GatedRotaryMixer}
 
 MIXERS = {"attention": BiasedAttentionMixer, "channel_delta": ChannelDeltaMixer,
           "rotary_window": RotaryWindowAttentionMixer,
@@ -1133,18 +1238,29 @@ class ParallelLayer(nn.Module):
     outputs and the activated feed-forward are columns of one buffer and
     out_w joins their output projections, so the sum over the sublayers is the
     accumulation of a single product. A mixer that also reads the previous
-    token's h gets its mixed inputs as further planes beside h."""
+    token's h gets its mixed inputs as further planes beside h.
+
+    Style "parallel_rms": the feed-forward reads an RMS norm of its own
+    (plane 1), act(gate) * up with gate and up rows alternating in in_w."""
 
     def __init__(self, spec: HybridSpec, ls: HybridLayerSpec, dtype, gen):
         super().__init__()
         C, dev = spec.hidden_size, gen.device
-        self.C, self.dtype = C, dtype
-        self.norm1 = DyTNorm(C, gen)
+        self.C, self.dtype, self.eps = C, dtype, spec.norm_eps
+        self.rms = spec.layer_style == "parallel_rms"
+        if self.rms:
+            # weights of the mixer's and the feed-forward's norm, less one
+            self.norms_w = _param(0.05 * _rand(gen, 1 if ls.mlp_kind is None else 2, C))
+        else:
+            self.norm1 = DyTNorm(C, gen)
         self.mixer = PART_MIXERS[ls.mixer.kind](C, ls.mixer, spec.norm_eps, dtype, gen)
         rows = [r for r in self.mixer.inputs()]
         cols = list(self.mixer.outputs)
         if ls.mlp_kind == "dense":
-            rows.append(InputRows("up", ls.mlp_ff, ["up"], 0, ls.mlp_act))
+            if self.rms:
+                rows.append(InputRows("up", 2 * ls.mlp_ff, ["gate", "up"], 1, ls.mlp_act, True))
+            else:
+                rows.append(InputRows("up", ls.mlp_ff, ["up"], 0, ls.mlp_act))
             cols.append(("up", ls.mlp_ff))
         elif ls.mlp_kind is not None:
             raise ValueError(f"parallel layers take dense feed-forwards, not {ls.mlp_kind!r}")
@@ -1152,7 +1268,7 @@ class ParallelLayer(nn.Module):
         self.rows = sorted(rows, key=lambda r: r.plane)      # stable: equal planes adjacent
         self.groups, at = [], 0
         for r in self.rows:
-            self.groups.append(mx.RowGroup(at, at + _pad16(r.rows), r.plane, r.act))
+            self.groups.append(mx.RowGroup(at, at + _pad16(r.rows), r.plane, r.act, r.paired))
             at += _pad16(r.rows)
         self.in_w = _param(_rand(gen, at, C, std=1.0 / math.sqrt(C), dtype=dtype))
         self.cols, at, live = [], 0, 0
@@ -1173,6 +1289,8 @@ class ParallelLayer(nn.Module):
         self.mu = None
         if self.mixer.mu_names:
             self.mu = _param(torch.rand(len(self.mixer.mu_names), C, generator=gen, device=dev))
+        if self.rms and (self.mu is not None or self.out_b is not None):
+            raise ValueError("parallel_rms layers take mixers without token shift and output bias")
 
     def state_shapes(self) -> Dict[str, tuple]:
         shapes = dict(self.mixer.state_shapes())
@@ -1182,7 +1300,9 @@ class ParallelLayer(nn.Module):
 
     def enter(self, x, sb: mx.SeqBatch, state, y=None, bias=None, extra=None) -> torch.Tensor:
         """Adds what the previous layer left over (y, bias, extra) to the
-        residual x and returns this layer's inputs [1 + mixes, T, C]."""
+        residual x and returns this layer's inputs [planes, T, C]."""
+        if self.rms:
+            return mx.add_rms_norm(x, self.norms_w, self.eps, self.dtype, y=y, offset=1.0)
         P = 1 if self.mu is None else 1 + self.mu.shape[0]
         hs = torch.empty(P, x.shape[0], self.C, dtype=self.dtype, device=x.device)
         norm = self.norm1.params()
@@ -1205,17 +1325,26 @@ class ParallelLayer(nn.Module):
         if self.has_ff:
             i = [r.key for r in self.rows].index("up")
             lo = self.cols[-1][1]
-            targets[i] = cat[:, lo : lo + _pad16(self.rows[i].rows)]
+            targets[i] = cat[:, lo : lo + self.groups[i].width]
         parts = mx.grouped_linear(hs, self.in_w, self.groups, targets)
         p = {r.key: t[:, : r.rows] for r, t in zip(self.rows, parts)}
         self.mixer(p, sb, kv, state, outs)
         return mx.linear_partials(cat, self.out_w)
 
     def load(self, get, put, p: str) -> None:
-        self.norm1.load(get, put, p + "norm1")
+        if self.rms:
+            put(self.norms_w, [get(p + n).reshape(1, -1) for n in ("norm1", "norm2")[: len(self.norms_w)]])
+        else:
+            self.norm1.load(get, put, p + "norm1")
+        source_rows = getattr(self.mixer, "source_rows", None)
         for r, g in zip(self.rows, self.groups):
             q = p + ("mlp." if r.key == "up" else "mix.")
-            put(self.in_w[g.begin : g.begin + r.rows], [get(q + s) for s in r.sources])
+            parts = [get(q + s) for s in r.sources]
+            if r.paired:
+                parts = [torch.stack(parts, 1).reshape(r.rows, -1)]
+            elif source_rows is not None and r.key != "up":
+                parts = [source_rows(s, w) for s, w in zip(r.sources, parts)]
+            put(self.in_w[g.begin : g.begin + r.rows], parts)
         for key, lo, n in self.cols:
             name = p + "mlp.down" if key == "up" else p + "mix." + key
             put(self.out_w[:, lo : lo + n], [get(name)])
@@ -1228,7 +1357,7 @@ class ParallelLayer(nn.Module):
 
 
 LAYER_STYLES = {"post_canon": HybridLayer, "sandwich": SandwichLayer, "pre_norm": PreNormLayer,
-                "hyper": HyperLayer, "parallel": ParallelLayer}
+                "hyper": HyperLayer, "parallel": ParallelLayer, "parallel_rms": ParallelLayer}
 
 
 class HybridForCausalLM(nn.Module):
@@ -1247,7 +1376,8 @@ class HybridForCausalLM(nn.Module):
         self.sandwich = spec.layer_style == "sandwich"
         self.pre_norm = spec.layer_style == "pre_norm"
         self.hyper = spec.layer_style == "hyper"
-        self.parallel = spec.layer_style == "parallel"
+        self.rms = spec.layer_style == "parallel_rms"
+        self.parallel = spec.layer_style == "parallel" or self.rms
         # the order the layers run in (a looped layer once per pass); caches
         # and state are kept per RUN, weights per layer
         self.runs = spec.layer_runs()
@@ -1255,7 +1385,12 @@ class HybridForCausalLM(nn.Module):
         self.layers = nn.ModuleList(
             [LAYER_STYLES[spec.layer_style](spec, ls, dtype, gen) for ls in spec.layers]
         )
-        if self.sandwich or self.parallel:
+        self.embed_norm_w = None
+        if spec.embed_norm:
+            self.embed_norm_w = _param(0.05 * _rand(gen, 1, C))
+        if self.rms:
+            self.final_norm_w = _param(torch.zeros(1, C, device=device))
+        elif self.sandwich or self.parallel:
             self.final_norm = DyTNorm(C, gen)
         elif self.hyper:
             self.final_norm_w = _param(torch.ones(C, device=device))
@@ -1270,6 +1405,10 @@ class HybridForCausalLM(nn.Module):
         # layer i reads the cache of layer kv_source[i] (its own unless its
         # mixer names another layer)
         self.kv_source = [getattr(layer.mixer, "kv_source", None) for layer in self.layers]
+        # run r also reads the values that layer v_first[r] cached for its tokens
+        self.v_first = [getattr(self.layers[i].mixer, "v_first_from", None) for i in self.runs]
+        if any(v is not None for v in self.v_first) and spec.loop:
+            raise ValueError("values of an earlier layer are not defined over looped layers")
         if spec.tied_head:
             self.lm_head = self.embed           # the head IS the embedding table
         else:
@@ -1293,19 +1432,25 @@ class HybridForCausalLM(nn.Module):
         sb = fb.seq_batch
         assert sb is not None and state is not None, "hybrid models run flat multi-sequence steps"
         x = mx.embed_rows(self.embed, fb.input_ids, self.spec.embed_scale, self.pos_freq, sb)
+        if self.embed_norm_w is not None:
+            x = mx.add_rms_norm(x, self.embed_norm_w, self.spec.norm_eps, torch.float32,
+                                offset=1.0)[0]
         if self.parallel:
             e0 = x.clone() if self.loop_entries else None
             y = bias = None
             for r, i in enumerate(self.runs):
                 layer = self.layers[i]
                 hs = layer.enter(x, sb, state[r], y, bias, e0 if r in self.loop_entries else None)
-                y, bias = layer(hs, sb, kv_caches[r], state[r]), layer.out_b
+                kv = kv_caches[r]
+                if self.v_first[r] is not None:
+                    kv = (*kv, kv_caches[self.v_first[r]][1])
+                y, bias = layer(hs, sb, kv, state[r]), layer.out_b
                 if self.trace_layers is not None:
-                    mx.dyt_norm(x, None, self.dtype, y=y, bias=bias)
+                    self._add(x, y, bias)
                     self.trace_layers.append(x.clone())
                     y = bias = None
             if y is not None:
-                mx.dyt_norm(x, None, self.dtype, y=y, bias=bias)
+                self._add(x, y, bias)
             return x
         if self.hyper:
             S, eps = self.spec.streams, self.spec.norm_eps
@@ -1339,10 +1484,20 @@ class HybridForCausalLM(nn.Module):
                 self.trace_layers.append(x.clone())
         return x  # float32 residual [T, C]; compute_logits norms the rows it needs
 
+    def _add(self, x, y, bias) -> None:
+        """x += y + bias in place; y may be partial planes (parallel styles)."""
+        if self.rms:
+            mx.add_rms_norm(x, None, self.spec.norm_eps, self.dtype, y=y)
+        else:
+            mx.dyt_norm(x, None, self.dtype, y=y, bias=bias)
+
     def compute_logits(self, hidden: torch.Tensor) -> torch.Tensor:
         """hidden: float32 residual rows. Returns float32 logits (soft-capped
         if the design caps them)."""
-        if self.sandwich or self.parallel:
+        if self.rms:
+            normed = mx.add_rms_norm(hidden.contiguous(), self.final_norm_w, self.spec.norm_eps,
+                                     self.dtype, offset=1.0)[0]
+        elif self.sandwich or self.parallel:
             normed = mx.dyt_norm(hidden.contiguous(), self.final_norm.params(), self.dtype)
         elif self.hyper:
             normed = mx.hyper_norm(hidden.contiguous().unsqueeze(1), self.one_read,
@@ -1393,10 +1548,14 @@ class HybridForCausalLM(nn.Module):
                 layer.load(get, put, f"l{i}.")
             return n
         if self.sandwich or self.pre_norm or self.parallel:
-            if not self.pre_norm:
+            if self.rms:
+                put(self.final_norm_w, [get("final.norm").reshape(1, -1)])
+            elif not self.pre_norm:
                 self.final_norm.load(get, put, "final.norm")
             else:
                 put(self.final_norm_w, [get("final.norm")])
+            if self.embed_norm_w is not None:
+                put(self.embed_norm_w, [get("embed.norm").reshape(1, -1)])
             for i, layer in enumerate(self.layers):
                 layer.load(get, put, f"l{i}.")
             return n

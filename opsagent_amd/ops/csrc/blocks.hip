@@ -162,10 +162,15 @@ extern "C" int oa_dyt_norm(void* stream, const void* y, int64_t ys, int ny, int6
 // channels from 2*nfreq on pass unrotated (qw and kw null: no norm, rotation
 // only). q goes to q_out [T, H, D], k and the unchanged v (Gv value heads of
 // Dv channels after the G key heads) to their cache slot. The position of token t of sequence b is past[b] + t - cu[b].
-// Everything between load and store is float32. A lane keeps its pairs in
-// bias (null: none) is added to the query and key columns first; Gv = 0: the
-// projection has no value columns and no value is written (attention whose
-// values are its keys).
+// Everything between load and store is float32.
+// bias (null: none) is added to the query and key columns first, vbias to the
+// value columns; Gv = 0: the projection has no value columns and no value is
+// written (attention whose values are its keys).
+// post (with qw, kw null): heads are divided by their root mean square after the
+// rotation instead, without a weight. mag multiplies cos and sin of the
+// rotated pairs. vfirst given: v <- (1 - lam) v + lam v_first, lam one float
+// in device memory, v_first the token's row of another layer's value cache.
+// A lane keeps its pairs in
 // registers (RP_NP pairs: D <= 128 * RP_NP), so every element is read once;
 // the token's cos/sin table is computed once per block into LDS.
 // PAIRED: D, the row stride and the head offsets are even, pairs are loaded
@@ -195,7 +200,8 @@ __global__ __launch_bounds__(256) void attn_rope_prepare_kernel(
     TC* __restrict__ q_out, TC* __restrict__ k_cache, TC* __restrict__ v_cache,
     const int* __restrict__ slot_mapping, const int* __restrict__ seq_of,
     const int* __restrict__ cu, const int* __restrict__ past, int B, int H, int G, int Gv, int D,
-    int Dv, float eps) {
+    int Dv, float eps, const TC* __restrict__ vbias, int post, float mag,
+    const TC* __restrict__ vfirst, const float* __restrict__ lam) {
     const int t = blockIdx.x;
     if (t >= cu[B]) return;  // padding row of a fixed-size (captured) launch
     const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
@@ -210,7 +216,11 @@ __global__ __launch_bounds__(256) void attn_rope_prepare_kernel(
     float* sn = lds + npair;    // [npair]
     for (int i = threadIdx.x; i < npair; i += blockDim.x) {
         float s_ = 0.0f, c_ = 1.0f;
-        if (i < nfreq) sincosf(pos * inv_freq[i], &s_, &c_);
+        if (i < nfreq) {
+            sincosf(pos * inv_freq[i], &s_, &c_);
+            c_ *= mag;
+            s_ *= mag;
+        }
         cs[i] = c_;
         sn[i] = s_;
     }
@@ -246,12 +256,22 @@ __global__ __launch_bounds__(256) void attn_rope_prepare_kernel(
         for (int k = 0; k < RP_HU; ++k) {
             const int hd = h0 + k;
             if (hd >= nh) continue;                // uniform over the wave
+            const bool is_q = hd < H;
+            if (post) {                            // the norm follows: rotate first
+#pragma unroll
+                for (int j = 0; j < RP_NP; ++j) {
+                    const int i = lane + 64 * j;
+                    if (i >= npair) continue;
+                    const float a = u[k][j], c = v[k][j];
+                    u[k][j] = a * cs[i] - c * sn[i];
+                    v[k][j] = c * cs[i] + a * sn[i];
+                }
+            }
             float ss = 0.0f;
 #pragma unroll
             for (int j = 0; j < RP_NP; ++j) ss += u[k][j] * u[k][j] + v[k][j] * v[k][j];
             ss = wave_reduce_sum(ss);
-            const float rn = qw ? 1.0f / sqrtf(ss / (float)D + eps) : 1.0f;
-            const bool is_q = hd < H;
+            const float rn = qw || post ? 1.0f / sqrtf(ss / (float)D + eps) : 1.0f;
             TC* dst = is_q ? q_out + ((int64_t)t * H + hd) * D
                            : k_cache + (slot * G + (hd - H)) * D;
 #pragma unroll
@@ -259,10 +279,10 @@ __global__ __launch_bounds__(256) void attn_rope_prepare_kernel(
                 const int i = lane + 64 * j;
                 if (i >= npair) continue;
                 const float* w = is_q ? qw : kw;
-                const float a = w ? u[k][j] * rn * w[2 * i] : u[k][j];
-                const float c = (2 * i + 1 < D) ? (w ? v[k][j] * rn * w[2 * i + 1] : v[k][j]) : 0.0f;
-                const float ra = a * cs[i] - c * sn[i];
-                const float rc = c * cs[i] + a * sn[i];
+                const float a = w ? u[k][j] * rn * w[2 * i] : u[k][j] * rn;
+                const float c = (2 * i + 1 < D) ? (w ? v[k][j] * rn * w[2 * i + 1] : v[k][j] * rn) : 0.0f;
+                const float ra = post ? a : a * cs[i] - c * sn[i];
+                const float rc = post ? c : c * cs[i] + a * sn[i];
                 if (PAIRED) {
                     st2(dst, 2 * i, ra, rc);
                 } else {
@@ -272,11 +292,19 @@ __global__ __launch_bounds__(256) void attn_rope_prepare_kernel(
             }
         }
     }
-    // values: a plain copy of Gv*Dv contiguous columns to the token's slot
+    // values: Gv*Dv contiguous columns to the token's slot
     const TC* vsrc = row + (int64_t)nh * D;
     TC* vdst = v_cache + slot * (int64_t)(Gv * Dv);
     const int nv = Gv * Dv, tid = blockIdx.y * blockDim.x + threadIdx.x, nt = gridDim.y * blockDim.x;
-    if (PAIRED) {
+    if (vbias || vfirst) {
+        const TC* fsrc = vfirst ? vfirst + slot * (int64_t)nv : nullptr;
+        const float lm = vfirst ? lam[0] : 0.0f;
+        for (int i = tid; i < nv; i += nt) {
+            float x = ldf(vsrc, i) + (vbias ? ldf(vbias, i) : 0.0f);
+            if (fsrc) x = (1.0f - lm) * x + lm * ldf(fsrc, i);
+            stf(vdst, i, x);
+        }
+    } else if (PAIRED) {
         for (int i = tid; 2 * i < nv; i += nt) {
             float a, c;
             ld2(vsrc, 2 * i, a, c);
@@ -302,7 +330,8 @@ __global__ __launch_bounds__(256) void attn_rope_prepare_vec_kernel(
     TC* __restrict__ q_out, TC* __restrict__ k_cache, TC* __restrict__ v_cache,
     const int* __restrict__ slot_mapping, const int* __restrict__ seq_of,
     const int* __restrict__ cu, const int* __restrict__ past, int B, int H, int G, int Gv, int D,
-    int Dv, float eps) {
+    int Dv, float eps, const TC* __restrict__ vbias, int post, float mag,
+    const TC* __restrict__ vfirst, const float* __restrict__ lam) {
     extern __shared__ float lds[];
     const int npair = D / 2;
     float* cs = lds;            // [npair]
@@ -314,7 +343,11 @@ __global__ __launch_bounds__(256) void attn_rope_prepare_vec_kernel(
     const float pos = (float)(past[b] + t - cu[b]);
     for (int i = threadIdx.x; i < npair; i += blockDim.x) {
         float s_ = 0.0f, c_ = 1.0f;
-        if (i < nfreq) sincosf(pos * inv_freq[i], &s_, &c_);
+        if (i < nfreq) {
+            sincosf(pos * inv_freq[i], &s_, &c_);
+            c_ *= mag;
+            s_ *= mag;
+        }
         cs[i] = c_;
         sn[i] = s_;
     }
@@ -355,12 +388,21 @@ __global__ __launch_bounds__(256) void attn_rope_prepare_vec_kernel(
 #pragma unroll
         for (int k = 0; k < RV_IT; ++k) {
             const int hd = h0 + k * step;
+            if (post) {                              // the norm follows: rotate first
+#pragma unroll
+                for (int e = 0; e < 8; e += 2) {
+                    const float a = x[k][e], c = x[k][e + 1];
+                    const float cc = cs[(ch + e) >> 1], sv = sn[(ch + e) >> 1];
+                    x[k][e] = a * cc - c * sv;
+                    x[k][e + 1] = c * cc + a * sv;
+                }
+            }
             float ss = 0.0f;
 #pragma unroll
             for (int e = 0; e < 8; ++e) ss += x[k][e] * x[k][e];
             for (int off = lph >> 1; off > 0; off >>= 1) ss += __shfl_xor(ss, off, WAVE);
             if (hd >= nh) continue;
-            const float rn = qw ? 1.0f / sqrtf(ss / (float)D + eps) : 1.0f;
+            const float rn = qw || post ? 1.0f / sqrtf(ss / (float)D + eps) : 1.0f;
             const bool is_q = hd < H;
             float o[8];
 #pragma unroll
@@ -368,8 +410,8 @@ __global__ __launch_bounds__(256) void attn_rope_prepare_vec_kernel(
                 const float a = x[k][e] * rn * (is_q ? wq[e] : wk[e]);
                 const float c = x[k][e + 1] * rn * (is_q ? wq[e + 1] : wk[e + 1]);
                 const float cc = cs[(ch + e) >> 1], sv = sn[(ch + e) >> 1];
-                o[e] = a * cc - c * sv;
-                o[e + 1] = c * cc + a * sv;
+                o[e] = post ? a : a * cc - c * sv;
+                o[e + 1] = post ? c : c * cc + a * sv;
             }
             if (is_q) st8(q_out, ((int64_t)t * H + hd) * D + ch, o);
             else st8(k_cache, (slot * G + (hd - H)) * D + ch, o);
@@ -379,8 +421,19 @@ __global__ __launch_bounds__(256) void attn_rope_prepare_vec_kernel(
     TC* vdst = v_cache + slot * (int64_t)(Gv * Dv);
     const int nv = Gv * Dv;
     for (int i = (blockIdx.y * blockDim.x + threadIdx.x) * 8; i < nv; i += gridDim.y * blockDim.x * 8) {
-        float tmp[8];
+        float tmp[8], f[8];
         ld8(vsrc, i, tmp);
+        if (vbias) {
+            ld8(vbias, i, f);
+#pragma unroll
+            for (int e = 0; e < 8; ++e) tmp[e] += f[e];
+        }
+        if (vfirst) {
+            const float lm = lam[0];
+            ld8(vfirst, slot * (int64_t)nv + i, f);
+#pragma unroll
+            for (int e = 0; e < 8; ++e) tmp[e] = (1.0f - lm) * tmp[e] + lm * f[e];
+        }
         st8(vdst, i, tmp);
     }
 }
@@ -390,10 +443,13 @@ extern "C" int oa_attn_rope_prepare(void* stream, const void* qkv, int64_t qs, c
                                     void* q_out, void* k_cache, void* v_cache,
                                     const void* slot_mapping, const void* seq_of, const void* cu,
                                     const void* past, int B, int T, int H, int G, int Gv, int D,
-                                    int Dv, float eps, int dt) {
+                                    int Dv, float eps, int dt, const void* vbias, int post,
+                                    float mag, const void* vfirst, const void* lam) {
     // qw, kw both null: no norm, rotation only. Gv value heads follow the key heads
-    // (0: none). bias [H*D + G*D] in the activation type, or null.
+    // (0: none). bias [H*D + G*D] and vbias [Gv*Dv] in the activation type, or null.
+    // vfirst: a value cache of v_cache's shape and type, or null.
     if (T <= 0) return 0;
+    if ((post && qw) || (vfirst && !lam) || (Gv == 0 && (vbias || vfirst))) return -101;
     if (2 * nfreq > D || H < 1 || G < 1 || Gv < 0 || D > 128 * RP_NP || (qw == nullptr) != (kw == nullptr))
         return -100;
     hipStream_t s = (hipStream_t)stream;
@@ -409,7 +465,8 @@ extern "C" int oa_attn_rope_prepare(void* stream, const void* qkv, int64_t qs, c
     (const TC*)qkv, qs, (const TC*)bias, (const float*)qw, (const float*)kw,                   \
         (const float*)inv_freq, nfreq,                                                         \
         (TC*)q_out, (TC*)k_cache, (TC*)v_cache, (const int*)slot_mapping, (const int*)seq_of,  \
-        (const int*)cu, (const int*)past, B, H, G, Gv, D, Dv, eps
+        (const int*)cu, (const int*)past, B, H, G, Gv, D, Dv, eps, (const TC*)vbias, post, mag, \
+        (const TC*)vfirst, (const float*)lam
 #define RP(TC)                                                                                 \
     do {                                                                                       \
         if (paired) hipLaunchKernelGGL((attn_rope_prepare_kernel<TC, true>), dim3(T, ny),      \
@@ -422,7 +479,8 @@ extern "C" int oa_attn_rope_prepare(void* stream, const void* qkv, int64_t qs, c
     const bool vec8 = D % 8 == 0 && lph >= 1 && lph <= 64 && (lph & (lph - 1)) == 0 && Dv % 8 == 0 &&
                       qs % 8 == 0 && (uintptr_t)qkv % al == 0 && (uintptr_t)q_out % al == 0 &&
                       (uintptr_t)k_cache % al == 0 && (uintptr_t)v_cache % al == 0 &&
-                      (uintptr_t)qw % 16 == 0 && (uintptr_t)kw % 16 == 0 && (uintptr_t)bias % al == 0;
+                      (uintptr_t)qw % 16 == 0 && (uintptr_t)kw % 16 == 0 && (uintptr_t)bias % al == 0 &&
+                      (uintptr_t)vbias % al == 0 && (uintptr_t)vfirst % al == 0;
     if (vec8) {
         const int hpw = 64 / lph;
         const int vy = std::max(1, std::min(CEIL_DIV(H + G, 4 * hpw), 1024 / T));
@@ -521,6 +579,54 @@ extern "C" int oa_act_mul_rows(void* stream, const void* gu, void* out, int64_t 
             hipLaunchKernelGGL((act_mul_rows_kernel<bf16s>), dim3(grid), dim3(256), 0, s,
                                (const bf16s*)gu, (bf16s*)out, M, I, act, limit, alpha);
     }
+    HIP_CHECK_LAUNCH();
+    return 0;
+}
+
+// The same over rows of alternating gate and up columns (g_0, u_0, g_1, u_1, ..):
+// out[m, i] = act(x[m, 2 i]) * x[m, 2 i + 1]. Both row strides are free. VEC:
+// 4 outputs per thread.
+template <typename TC, bool VEC>
+__global__ __launch_bounds__(256) void act_pair_rows_kernel(const TC* __restrict__ x, int64_t xs,
+                                                            TC* __restrict__ out, int64_t os,
+                                                            int64_t M, int I, int act) {
+    constexpr int W = VEC ? 4 : 1;
+    const uint32_t iv = I / W, total = (uint32_t)M * iv;          // fits: checked by the host
+    for (uint32_t i = blockIdx.x * blockDim.x + threadIdx.x; i < total; i += gridDim.x * blockDim.x) {
+        const int64_t m = i / iv;
+        const int c = (int)(i % iv) * W;
+        if (VEC) {
+            float a[8], o[4];
+            ld8(x, m * xs + 2 * c, a);
+#pragma unroll
+            for (int e = 0; e < 4; ++e) o[e] = gate_act_f(a[2 * e], act) * a[2 * e + 1];
+            stq4(out, m * os + c, o);
+        } else {
+            stf(out, m * os + c, gate_act_f(ldf(x, m * xs + 2 * c), act) * ldf(x, m * xs + 2 * c + 1));
+        }
+    }
+}
+
+extern "C" int oa_act_pair_rows(void* stream, const void* x, int64_t xs, void* out, int64_t os,
+                                int64_t M, int I, int dt, int act) {
+    if (M <= 0 || I <= 0) return 0;
+    if (act < 0 || act > 1 || xs < 2 * (int64_t)I || os < I) return -100;
+    if (M * I > 0xf0000000LL) return -101;
+    hipStream_t s = (hipStream_t)stream;
+    const int al = dt == 1 ? 32 : 16;
+    const bool vec = I % 4 == 0 && xs % 8 == 0 && os % 4 == 0 && (uintptr_t)x % al == 0 &&
+                     (uintptr_t)out % (al / 2) == 0;
+#define AP_LAUNCH(TC, V)                                                                         \
+    hipLaunchKernelGGL((act_pair_rows_kernel<TC, V>), dim3(grid_for(M * (V ? I / 4 : I))), dim3(256), \
+                       0, s, (const TC*)x, xs, (TC*)out, os, M, I, act)
+    if (dt == 1) {
+        if (vec) AP_LAUNCH(float, true);
+        else AP_LAUNCH(float, false);
+    } else {
+        if (vec) AP_LAUNCH(bf16s, true);
+        else AP_LAUNCH(bf16s, false);
+    }
+#undef AP_LAUNCH
     HIP_CHECK_LAUNCH();
     return 0;
 }

@@ -564,13 +564,14 @@ extern "C" int oa_gemv_bf16_mfma(void* stream, const void* x, const void* w,
 // group g = rows [begin, end), reads activation plane `plane` of x [P, M, K]
 // and writes act(row . x) to column row - begin of its own output rows.
 // begin and end are multiples of 16, so neither the two adjacent rows of a
-// wave nor the 16 rows of a matrix-core tile straddle a group.
+// wave nor the 16 rows of a matrix-core tile straddle a group. In a paired group
+// gate and up rows alternate and (row - begin) / 2 takes act(gate) * up.
 #define GEMV_MAX_GROUPS 8
 struct GemvGroups {
     int n;
     int end[GEMV_MAX_GROUPS];
     int plane[GEMV_MAX_GROUPS];
-    int act[GEMV_MAX_GROUPS];         // 0 none, 1 silu, 2 gelu (tanh form)
+    int act[GEMV_MAX_GROUPS];         // 0 none, 1 silu, 2 gelu (tanh form); + 4: paired
     uint16_t* out[GEMV_MAX_GROUPS];
     int64_t os[GEMV_MAX_GROUPS];      // elements between the output rows
 };
@@ -583,6 +584,7 @@ __device__ __forceinline__ int gemv_group_of(const GemvGroups& g, int row) {
 __device__ __forceinline__ float gemv_group_act(float v, int act) {
     return act ? gate_act(v, act - 1) : v;
 }
+#define GEMV_PAIRED 4
 
 template <int M, int RW>
 __global__ __launch_bounds__(256) void gemv_grouped_kernel(const uint32_t* __restrict__ x,
@@ -620,6 +622,16 @@ __global__ __launch_bounds__(256) void gemv_grouped_kernel(const uint32_t* __res
         }
         const int c0 = row0 - (gi ? gr.end[gi - 1] : 0);
         uint16_t* out = gr.out[gi];
+        if (RW == 2 && (gr.act[gi] & GEMV_PAIRED)) {
+#pragma unroll
+            for (int m = 0; m < M; ++m) {
+                const float g = wave_reduce_sum(acc[0][m]), u = wave_reduce_sum(acc[RW - 1][m]);
+                if (lane == 0)
+                    out[(size_t)m * gr.os[gi] + c0 / 2] =
+                        f32_to_bf16(gemv_group_act(g, gr.act[gi] - GEMV_PAIRED) * u);
+            }
+            continue;
+        }
 #pragma unroll
         for (int m = 0; m < M; ++m)
 #pragma unroll
@@ -703,6 +715,13 @@ __global__ __launch_bounds__(256, 1) void gemv_grouped_mfma_kernel(
         return;
     }
     const int c0 = row0 - (gi ? gr.end[gi - 1] : 0);
+    if (gr.act[gi] & GEMV_PAIRED) {
+        uint16_t* po = gr.out[gi] + (size_t)fr * gr.os[gi] + c0 / 2 + fs * 2;
+        const int act = gr.act[gi] - GEMV_PAIRED;
+#pragma unroll
+        for (int i = 0; i < 2; ++i) po[i] = f32_to_bf16(gemv_group_act(v[2 * i], act) * v[2 * i + 1]);
+        return;
+    }
     uint16_t* out = gr.out[gi] + (size_t)fr * gr.os[gi] + c0 + fs * 4;
 #pragma unroll
     for (int i = 0; i < 4; ++i) out[i] = f32_to_bf16(gemv_group_act(v[i], gr.act[gi]));
@@ -733,10 +752,13 @@ extern "C" int oa_gemv_grouped(void* stream, const void* x, const void* w, int M
     GemvGroups gr;
     gr.n = n;
     int prev = 0;
+    bool paired = false;
     for (int i = 0; i < n; ++i) {
-        if (end[i] <= prev || end[i] % 16 != 0 || plane[i] < 0 || act[i] < 0 || act[i] > 2 || !out[i] ||
-            os[i] < end[i] - prev)
+        const int kind = act[i] & ~GEMV_PAIRED, pair = act[i] & GEMV_PAIRED ? 1 : 0;
+        if (end[i] <= prev || end[i] % 16 != 0 || plane[i] < 0 || kind < 0 || kind > 2 || !out[i] ||
+            os[i] < (end[i] - prev) >> pair)
             return -101;
+        paired |= pair;
         gr.end[i] = prev = end[i];
         gr.plane[i] = plane[i];
         gr.act[i] = act[i];
@@ -754,7 +776,7 @@ extern "C" int oa_gemv_grouped(void* stream, const void* x, const void* w, int M
         HIP_CHECK_LAUNCH();
         return 0;
     }
-    const bool rw1 = N <= 6144;
+    const bool rw1 = N <= 6144 && !paired;
     const int grid = std::min(2048, CEIL_DIV(N, rw1 ? 4 : 8));
 #define GG(MV)                                                                                     \
     do {                                                                                           \

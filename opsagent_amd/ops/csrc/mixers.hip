@@ -404,15 +404,16 @@ __global__ __launch_bounds__(256) void attn_prepare_vec_kernel(
 //   score(i, j) = q_i . k_j * scale - slope_h * (i - j),  j <= i
 //                 (slopes null: no distance penalty)
 //   window > 0: only keys j > i - window are visible (the last `window`
-//                 positions up to the query); key tiles that end before
-//                 that range are never visited
+//                 positions up to the query) and the keys j < keep_first;
+//                 key tiles that hold neither are never visited
 //   softcap > 0: q_i . k_j * scale is replaced by softcap * tanh(that / softcap)
 //   Gv value heads (Gv divides G): key head g reads value head g mod Gv
 //   sinks given: Z_i,h = sum_j exp(score(i, j)) + exp(sink_h): the sink
 //                 enlarges the normaliser only, contributes no value
 //                 vector, and `scale` is not applied to it
 //   out_i,h = oscale * (sigmoid(gate_i,h)) * sum_j softmax_j(score) v_j
-//                 (gate null: 1), token rows `os` elements apart
+//                 (gate null: 1; gch: one gate per output channel,
+//                 gate_i,h,c), token rows `os` elements apart
 // grid = (query tiles, kv heads, key splits). A tile is up to TQ
 // consecutive new tokens of ONE sequence with all R = H/G query heads of
 // the kv head: ROWS = TQ*R rows share every staged key/value tile. Each of
@@ -424,6 +425,20 @@ __global__ __launch_bounds__(256) void attn_prepare_vec_kernel(
 #define ATT_MAXR 4   // rows per wave
 #define ATT_MAXV 4   // value channels per lane (Dv <= 256)
 
+// The key tiles a block visits, in ascending order: those that hold kept first
+// keys (as far as they lie before the window), then those of the window.
+struct KeyTiles {
+    int kept, first, count;
+    __device__ __forceinline__ int at(int i) const { return i < kept ? i : i - kept + first; }
+};
+__device__ __forceinline__ KeyTiles key_tiles(int first_pos, int nkt, int KT, int window, int keep) {
+    KeyTiles k;
+    k.first = window > 0 ? max(0, first_pos - window + 1) / KT : 0;
+    k.kept = min((keep + KT - 1) / KT, k.first);
+    k.count = k.kept + nkt - k.first;
+    return k;
+}
+
 template <typename TC>
 __global__ __launch_bounds__(256) void attn_bias_paged_kernel(
     const TC* __restrict__ q, const TC* __restrict__ gate, int64_t gs,
@@ -433,7 +448,7 @@ __global__ __launch_bounds__(256) void attn_bias_paged_kernel(
     const int* __restrict__ block_table, int max_blocks, int block_size,
     const float* __restrict__ slopes, const float* __restrict__ sinks, int B, int H, int G,
     int D, int Dv, int TQ, int KT, int kstride, float scale, int nsplit, int RB, int window,
-    int64_t vrow, int Gv, float softcap, int64_t os, float oscale) {
+    int64_t vrow, int Gv, float softcap, int64_t os, float oscale, int keep, int gch) {
     extern __shared__ float lds[];
     // a block takes up to RB of the H/G query heads of one kv head
     const int hgroups = (H / G + RB - 1) / RB;
@@ -477,11 +492,9 @@ __global__ __launch_bounds__(256) void attn_bias_paged_kernel(
 #pragma unroll
         for (int c = 0; c < ATT_MAXV; ++c) acc[i][c] = 0.0f;
     }
-    const int nkt = last_pos / KT + 1;
-    // the first key any query of the tile sees
-    const int kt_first = window > 0 ? max(0, p0 - window + 1) / KT : 0;
-    for (int kt = kt_first + split; kt < nkt; kt += nsplit) {
-        const int k0 = kt * KT;
+    const KeyTiles tiles = key_tiles(p0, last_pos / KT + 1, KT, window, keep);
+    for (int it = split; it < tiles.count; it += nsplit) {
+        const int k0 = tiles.at(it) * KT;
         const int nk = min(KT, last_pos + 1 - k0);
         __syncthreads();
         for (int i = threadIdx.x; i < nk * D; i += blockDim.x) {
@@ -503,10 +516,10 @@ __global__ __launch_bounds__(256) void attn_bias_paged_kernel(
             if (r >= rows) break;
             const int pos = p0 + r / R;
             const int kmin = window > 0 ? pos - window + 1 : 0;   // first key seen
-            if (k0 > pos || k0 + nk <= kmin) continue;
+            if (k0 > pos || (k0 + nk <= kmin && k0 >= keep)) continue;
             const float slope = slopes ? slopes[h0 + r % R] : 0.0f;
             float s = -INFINITY;
-            if (lane < nk && k0 + lane <= pos && k0 + lane >= kmin) {
+            if (lane < nk && k0 + lane <= pos && (k0 + lane >= kmin || k0 + lane < keep)) {
                 const float* qr = Qs + r * D;
                 const TC* kr = Ks + lane * kstride;
                 float a = 0.0f;
@@ -542,13 +555,16 @@ __global__ __launch_bounds__(256) void attn_bias_paged_kernel(
         if (r >= rows) break;
         const int tok = lo + t0 + r / R, h = h0 + r % R;
         if (nsplit == 1) {
-            const float gt = gate ? sigmoidf_(ldf(gate, (int64_t)tok * gs + h)) : 1.0f;
+            const float gt = gate && !gch ? sigmoidf_(ldf(gate, (int64_t)tok * gs + h)) : 1.0f;
             const float lt = sinks ? l[ri] + expf(sinks[h] - m[ri]) : l[ri];
             const float inv = gt * oscale / lt;
 #pragma unroll
             for (int c = 0; c < ATT_MAXV; ++c) {
                 const int ch = lane + 64 * c;
-                if (ch < Dv) stf(out, (int64_t)tok * os + h * Dv + ch, acc[ri][c] * inv);
+                if (ch >= Dv) continue;
+                float v = acc[ri][c] * inv;
+                if (gate && gch) v *= sigmoidf_(ldf(gate, (int64_t)tok * gs + h * Dv + ch));
+                stf(out, (int64_t)tok * os + h * Dv + ch, v);
             }
         } else {
             const int64_t pr = ((int64_t)tok * H + h) * nsplit + split;
@@ -602,7 +618,7 @@ __global__ __launch_bounds__(256) void attn_bias_mfma_kernel(
     const int* __restrict__ block_table, int max_blocks, int block_size,
     const float* __restrict__ slopes, const float* __restrict__ sinks, int B, int H, int G,
     int D, int Dv, int HB, float scale, int nsplit, int window, int vrow, int hrows, int Gv,
-    float softcap, int64_t os, float oscale) {
+    float softcap, int64_t os, float oscale, int keep, int gch) {
     // hrows (decode steps of many query heads per kv head): a step brings one
     // token per sequence, so the 16 columns of a wave's tile are 16 HEADS at
     // that token's position instead of 16 tokens of one head; a block covers
@@ -734,11 +750,12 @@ __global__ __launch_bounds__(256) void attn_bias_mfma_kernel(
                                        : make_uint4(0, 0, 0, 0);
         }
     };
-    // key tiles before the window of the block's first query are skipped
-    const int kt_first = window > 0 ? max(0, pb + tile * TQ - window + 1) / MF_KT : 0;
-    if (kt_first + split < nkt) fetch(kt_first + split);
-    for (int kt = kt_first + split; kt < nkt; kt += nsplit) {
-        const int k0 = kt * MF_KT;
+    // key tiles before the window of the block's first query are skipped,
+    // except those that hold kept first keys
+    const KeyTiles tiles = key_tiles(pb + tile * TQ, nkt, MF_KT, window, keep);
+    if (split < tiles.count) fetch(tiles.at(split));
+    for (int it = split; it < tiles.count; it += nsplit) {
+        const int k0 = tiles.at(it) * MF_KT;
         __syncthreads();
 #pragma unroll
         for (int u = 0; u < KC; ++u) {
@@ -758,8 +775,9 @@ __global__ __launch_bounds__(256) void attn_bias_mfma_kernel(
             }
         }
         __syncthreads();
-        if (kt + nsplit < nkt) fetch(kt + nsplit);
-        if (wave_ntok <= 0 || k0 > wave_last || k0 + MF_KT - 1 <= pb + t0 - wlim) continue;
+        if (it + nsplit < tiles.count) fetch(tiles.at(it + nsplit));
+        if (wave_ntok <= 0 || k0 > wave_last || (k0 + MF_KT - 1 <= pb + t0 - wlim && k0 >= keep))
+            continue;
         // S^T tiles: keys k0 + 16*mt + 4*lg + r, token lc of sub-tile u
         f4_t sc[NT][4];
 #pragma unroll
@@ -816,7 +834,7 @@ __global__ __launch_bounds__(256) void attn_bias_mfma_kernel(
                     }
                     if (diag) {
                         const int key = k0 + 16 * mt + 4 * lg + r;
-                        v = (key <= pos[u] && key > pos[u] - wlim) ? v : -INFINITY;
+                        v = (key <= pos[u] && (key > pos[u] - wlim || key < keep)) ? v : -INFINITY;
                     }
                     sc[u][mt][r] = v;
                     mloc = fmaxf(mloc, v);
@@ -877,15 +895,22 @@ __global__ __launch_bounds__(256) void attn_bias_mfma_kernel(
         const int tok = hrows ? lo : lo + t0 + 16 * u + lc;
         if (nsplit == 1) {
             const float lt = sinks ? l[u] + __builtin_amdgcn_exp2f(sinks[h] * LOG2E - m[u]) : l[u];
-            const float gt = (gate ? sigmoidf_(ldf(gate, (int64_t)tok * gs + h)) : 1.0f) * oscale / lt;
+            const float gt = (gate && !gch ? sigmoidf_(ldf(gate, (int64_t)tok * gs + h)) : 1.0f) * oscale / lt;
             bf16s* orow = out + (int64_t)tok * os + h * Dv + 4 * lg;
+            const bf16s* grow = gate + (int64_t)tok * gs + h * Dv + 4 * lg;
 #pragma unroll
             for (int dt = 0; dt < MAXDV; ++dt)
                 if (16 * dt < Dv) {
-                    uint2 w;
-                    w.x = pack_bf16x2(o[u][dt][0] * gt, o[u][dt][1] * gt);
-                    w.y = pack_bf16x2(o[u][dt][2] * gt, o[u][dt][3] * gt);
-                    *reinterpret_cast<uint2*>(orow + 16 * dt) = w;
+                    float v[4];
+#pragma unroll
+                    for (int r = 0; r < 4; ++r) v[r] = o[u][dt][r] * gt;
+                    if (gate && gch) {
+                        float gv[4];
+                        ldq4(grow, 16 * dt, gv);
+#pragma unroll
+                        for (int r = 0; r < 4; ++r) v[r] *= sigmoidf_(gv[r]);
+                    }
+                    stq4(orow, 16 * dt, v);
                 }
         } else {
             const int64_t pr = ((int64_t)tok * H + h) * nsplit + split;
@@ -907,7 +932,7 @@ template <typename TC>
 __global__ __launch_bounds__(64) void attn_combine_kernel(
     const float* __restrict__ part_o, const float* __restrict__ part_ml,
     const TC* __restrict__ gate, int64_t gs, const float* __restrict__ sinks,
-    TC* __restrict__ out, int H, int Dv, int nsplit, int64_t os, float oscale) {
+    TC* __restrict__ out, int H, int Dv, int nsplit, int64_t os, float oscale, int gch) {
     __shared__ float wsh[64];
     const int64_t row = blockIdx.x;  // tok * H + h
     const int tok = (int)(row / H), h = (int)(row % H);
@@ -923,7 +948,7 @@ __global__ __launch_bounds__(64) void attn_combine_kernel(
         mx = gmx;
     }
     if (sinks) lsum += expf(sinks[h] - mx);
-    const float gt = (gate ? sigmoidf_(ldf(gate, (int64_t)tok * gs + h)) : 1.0f) * oscale / lsum;
+    const float gt = (gate && !gch ? sigmoidf_(ldf(gate, (int64_t)tok * gs + h)) : 1.0f) * oscale / lsum;
     float acc[ATT_MAXV];
 #pragma unroll
     for (int c = 0; c < ATT_MAXV; ++c) acc[c] = 0.0f;
@@ -948,7 +973,10 @@ __global__ __launch_bounds__(64) void attn_combine_kernel(
 #pragma unroll
     for (int c = 0; c < ATT_MAXV; ++c) {
         const int ch = lane + 64 * c;
-        if (ch < Dv) stf(out, (int64_t)tok * os + h * Dv + ch, acc[c] * gt);
+        if (ch >= Dv) continue;
+        float v = acc[c] * gt;
+        if (gate && gch) v *= sigmoidf_(ldf(gate, (int64_t)tok * gs + h * Dv + ch));
+        stf(out, (int64_t)tok * os + h * Dv + ch, v);
     }
 }
 
@@ -1570,7 +1598,8 @@ static void launch_attn_mfma(hipStream_t s, dim3 grid, int lds_bytes, const void
                              const void* block_table, int max_blocks, int block_size,
                              const void* slopes, const void* sinks, int B, int H, int G, int D,
                              int Dv, int HB, float scale, int nsplit, int window, int64_t vrow,
-                             int hrows, int Gv, float softcap, int64_t os, float oscale) {
+                             int hrows, int Gv, float softcap, int64_t os, float oscale, int keep,
+                             int gch) {
     if (lds_bytes > 48 * 1024)
         (void)hipFuncSetAttribute((const void*)attn_bias_mfma_kernel<MAXD, MAXDV, QK32, NT>,
                                   hipFuncAttributeMaxDynamicSharedMemorySize, lds_bytes);
@@ -1579,7 +1608,7 @@ static void launch_attn_mfma(hipStream_t s, dim3 grid, int lds_bytes, const void
                        (const bf16s*)v_cache, (bf16s*)out, (float*)part_o, (float*)part_ml,
                        (const int*)cu, (const int*)past, (const int*)block_table, max_blocks,
                        block_size, (const float*)slopes, (const float*)sinks, B, H, G, D, Dv, HB,
-                       scale, nsplit, window, (int)vrow, hrows, Gv, softcap, os, oscale);
+                       scale, nsplit, window, (int)vrow, hrows, Gv, softcap, os, oscale, keep, gch);
 }
 
 // ntiles = sum_b ceil(n_b / TQ) (host-computed). part_* may be null when nsplit == 1.
@@ -1590,14 +1619,17 @@ extern "C" int oa_attn_bias_paged(void* stream, const void* q, const void* gate,
                                   const void* slopes, const void* sinks, int T, int B, int ntiles,
                                   int H, int G, int D, int Dv, float scale, int nsplit, int dt,
                                   int max_chunk, int window, int64_t vrow, int Gv, float softcap,
-                                  int64_t os, float oscale) {
+                                  int64_t os, float oscale, int keep, int gch) {
     // vrow: elements between the value rows of consecutive cache slots
     // (Gv * Dv for a cache of its own; more when the values are the leading
     // channels of wider rows). Gv value heads: key head g reads value head
     // g mod Gv. softcap > 0: score <- softcap * tanh(score / softcap).
     // os: elements between the output rows of consecutive tokens; oscale
-    // multiplies the output.
+    // multiplies the output. keep: keys below it are seen from beyond the window
+    // too. gch: gate rows hold H * Dv logits, one per output channel, instead
+    // of H.
     if (T <= 0 || ntiles <= 0) return 0;
+    if (keep < 0 || (gate && gs < (int64_t)H * (gch ? Dv : 1))) return -109;
     if (window < 0 || os < (int64_t)H * Dv) return -105;
     if (Gv < 1 || G % Gv != 0 || vrow < (int64_t)Gv * Dv) return -106;
     int TQ, KT, ks, lds_bytes;
@@ -1608,6 +1640,7 @@ extern "C" int oa_attn_bias_paged(void* stream, const void* q, const void* gate,
     if (attn_path(H, G, D, Dv, dt)) {
         if (vrow % 8 != 0) return -107;   // 16-byte value loads
         if (os % 4 != 0 || (uintptr_t)out % 8 != 0) return -108;   // 8-byte output stores
+        if (gate && gch && (gs % 4 != 0 || (uintptr_t)gate % 8 != 0)) return -110;   // and gate loads
         const int R = H / G, HB = attn_hb(R);
         // decode steps of 16 or more query heads per kv head put the heads
         // in the tile's columns
@@ -1616,7 +1649,7 @@ extern "C" int oa_attn_bias_paged(void* stream, const void* q, const void* gate,
 #define MF_ARGS                                                                                   \
     s, grid, lds_bytes, q, gate, gs, k_cache, v_cache, out, part_o, part_ml, cu, past, block_table, \
         max_blocks, block_size, slopes, sinks, B, H, G, D, Dv, HB, scale, nsplit, window, vrow, hrows, \
-        Gv, softcap, os, oscale
+        Gv, softcap, os, oscale, keep, gch
 #define MF(A, Bv)                                                               \
     do {                                                                        \
         if (D % 32 == 0) launch_attn_mfma<A, Bv, true, 1>(MF_ARGS);             \
@@ -1643,7 +1676,7 @@ extern "C" int oa_attn_bias_paged(void* stream, const void* q, const void* gate,
         (float*)part_o, (float*)part_ml, (const int*)cu, (const int*)past,                \
         (const int*)block_table, max_blocks, block_size, (const float*)slopes,            \
         (const float*)sinks, B, H, G, D, Dv, TQ, KT, ks, scale, nsplit, rb, window, vrow, Gv,  \
-        softcap, os, oscale
+        softcap, os, oscale, keep, gch
         if (dt == 1)
             hipLaunchKernelGGL((attn_bias_paged_kernel<float>), grid, blk, lds_bytes, s, AT_ARGS(float));
         else
@@ -1655,11 +1688,11 @@ extern "C" int oa_attn_bias_paged(void* stream, const void* q, const void* gate,
         if (dt == 1)
             hipLaunchKernelGGL((attn_combine_kernel<float>), dim3((unsigned)((int64_t)T * H)), dim3(64), 0, s,
                                (const float*)part_o, (const float*)part_ml, (const float*)gate, gs,
-                               (const float*)sinks, (float*)out, H, Dv, nsplit, os, oscale);
+                               (const float*)sinks, (float*)out, H, Dv, nsplit, os, oscale, gch);
         else
             hipLaunchKernelGGL((attn_combine_kernel<bf16s>), dim3((unsigned)((int64_t)T * H)), dim3(64), 0, s,
                                (const float*)part_o, (const float*)part_ml, (const bf16s*)gate, gs,
-                               (const float*)sinks, (bf16s*)out, H, Dv, nsplit, os, oscale);
+                               (const float*)sinks, (bf16s*)out, H, Dv, nsplit, os, oscale, gch);
         HIP_CHECK_LAUNCH();
     }
     return 0;

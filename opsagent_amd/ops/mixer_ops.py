@@ -229,15 +229,17 @@ def attention_paged(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tenso
                     window: Optional[int] = None,
                     sinks: Optional[torch.Tensor] = None,
                     softcap: Optional[float] = None, out_scale: float = 1.0,
-                    out: Optional[torch.Tensor] = None) -> torch.Tensor:
+                    out: Optional[torch.Tensor] = None, keep_first: int = 0,
+                    gate_channels: bool = False) -> torch.Tensor:
     """Causal softmax attention over each sequence's cached keys, score
     q.k*scale. Options, each a parameter: `slopes` [H] float32 subtracts
-    slope_h*(i-j); `window` hides keys with i - j >= window; `sinks` [H]
+    slope_h*(i-j); `window` hides keys with i - j >= window, except those at
+    positions j < `keep_first`; `sinks` [H]
     float32 enlarges head h's softmax normaliser by exp(sink_h) and leaves
     the numerator alone; `softcap` replaces the scaled score by
     softcap * tanh(score / softcap);
     `gate_logits` [T,H] (may be a column slice) scales each head's output by
-    its sigmoid; `out_scale` multiplies the result. q [T,H,D]. The cache may hold fewer value heads than key
+    its sigmoid, with `gate_channels` [T,H*Dv] each output channel; `out_scale` multiplies the result. q [T,H,D]. The cache may hold fewer value heads than key
     heads (Gv divides G): key head g reads value head g mod Gv.
     Returns [T, H*Dv]; `out` (rows of that width, may be a column slice of a
     wider buffer) takes the result if given."""
@@ -245,8 +247,11 @@ def attention_paged(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tenso
     nb, bs, Gv, Dv = v_cache.shape
     G = k_cache.shape[2]
     window = int(window) if window else 0
+    keep_first = int(keep_first) if window else 0
     softcap = float(softcap) if softcap else 0.0
     assert G % Gv == 0 and H % G == 0
+    assert gate_logits is None or (gate_logits.dtype == q.dtype and gate_logits.shape == (
+        T, H * Dv if gate_channels else H))
     # v_cache may be a view of the leading channels of wider rows (values
     # that are a prefix of the cached keys): its token stride is passed on
     assert v_cache.stride(3) == 1 and (Gv == 1 or v_cache.stride(2) == Dv)
@@ -254,7 +259,7 @@ def attention_paged(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tenso
     if not q.is_cuda:
         res = torch_ref.attention_paged(q, k_cache, v_cache, sb.cu, sb.past, sb.block_table,
                                         scale, slopes, gate_logits, window or None, sinks,
-                                        softcap or None)
+                                        softcap or None, keep_first, gate_channels)
         res = res * out_scale if out_scale != 1.0 else res
         return res if out is None else out.copy_(res)
     if Dv > ATTN_MAX_VALUES:
@@ -265,8 +270,12 @@ def attention_paged(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tenso
         wide = torch.empty(T, H, Dv, dtype=q.dtype, device=q.device)
         for lo in range(0, Dv, ATTN_MAX_VALUES):
             hi = min(Dv, lo + ATTN_MAX_VALUES)
-            part = attention_paged(q, k_cache, v_cache[..., lo:hi], sb, scale, slopes, gate_logits,
-                                   window, sinks, softcap, out_scale)
+            gate = gate_logits
+            if gate_logits is not None and gate_channels:
+                gate = gate_logits.reshape(T, H, Dv)[..., lo:hi].reshape(T, -1).contiguous()
+            part = attention_paged(q, k_cache, v_cache[..., lo:hi], sb, scale, slopes, gate,
+                                   window, sinks, softcap, out_scale, keep_first=keep_first,
+                                   gate_channels=gate_channels)
             wide[..., lo:hi] = part.view(T, H, hi - lo)
         wide = wide.view(T, H * Dv)
         return wide if out is None else out.copy_(wide)
@@ -277,7 +286,7 @@ def attention_paged(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tenso
     # few tiles and long contexts: split the keys over blocks to fill the chip
     reach = sb.max_total
     if window:
-        reach = min(reach, window + min(sb.max_chunk, TQ) + KT)
+        reach = min(reach, window + min(sb.max_chunk, TQ) + KT + (keep_first + KT - 1) // KT * KT)
     nkt = max(1, (reach + KT - 1) // KT)
     nsplit = 1
     if ntiles * G < 256 and nkt >= 8:
@@ -317,7 +326,7 @@ def attention_paged(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tenso
         sinks.data_ptr() if sinks is not None else None,
         T, sb.num_seqs, ntiles, H, G, D, Dv,
         float(scale), nsplit, dt, sb.max_chunk, window, v_cache.stride(1), Gv, softcap,
-        _rows(out), float(out_scale))
+        _rows(out), float(out_scale), keep_first, int(gate_channels))
     hip.check(rc, "oa_attn_bias_paged")
     return out
 
@@ -394,10 +403,26 @@ def rotary_inv_freq(dims: int, base: float, scaling: Optional[dict] = None) -> t
     {factor, low, high, original} slows long waves: a wavelength below
     original/high keeps its frequency, one above original/low gets
     frequency/factor, between them the two are blended linearly in
-    original/wavelength."""
+    original/wavelength. `scaling` {factor, fast, slow, original} (YaRN) blends
+    linearly in the pair's index i instead: with dim(t) = dims
+    ln(original / (2 pi t)) / (2 ln base) the index of the pair that makes t
+    turns over `original` positions, the frequency is kept up to
+    floor(dim(fast)) and divided by factor from ceil(dim(slow)) on."""
     import math
 
     out = []
+    yarn = bool(scaling) and "fast" in scaling
+    if yarn:
+        turns_dim = lambda t: (dims * math.log(float(scaling["original"]) / (2.0 * math.pi * t))  # noqa: E731
+                               / (2.0 * math.log(float(base))))
+        lo = max(math.floor(turns_dim(float(scaling["fast"]))), 0)
+        hi = min(math.ceil(turns_dim(float(scaling["slow"]))), dims - 1)
+        factor = float(scaling["factor"])
+        for i in range(dims // 2):
+            f = float(base) ** (-2.0 * i / dims)
+            ramp = min(max((i - lo) / max(hi - lo, 0.001), 0.0), 1.0)
+            out.append(f / factor * ramp + f * (1.0 - ramp))
+        return torch.tensor(out, dtype=torch.float32)
     for i in range(dims // 2):
         f = float(base) ** (-2.0 * i / dims)
         if scaling:
@@ -413,27 +438,51 @@ def rotary_inv_freq(dims: int, base: float, scaling: Optional[dict] = None) -> t
     return torch.tensor(out, dtype=torch.float32)
 
 
+def rotary_magnitude(scaling: Optional[dict] = None) -> float:
+    """What cos and sin of a rotation are multiplied by: 0.1 ln(factor) + 1
+    under the {factor, fast, slow, original} scaling, else 1."""
+    import math
+
+    if scaling and "fast" in scaling:
+        return 0.1 * math.log(float(scaling["factor"])) + 1.0
+    return 1.0
+
+
 def attn_rope_prepare(qkv: torch.Tensor, q_norm_w: Optional[torch.Tensor],
                       k_norm_w: Optional[torch.Tensor],
                       inv_freq: torch.Tensor, H: int, G: int, D: int, Dv: int, eps: float,
                       k_cache: torch.Tensor, v_cache: torch.Tensor, sb: SeqBatch,
                       v_heads: Optional[int] = None,
-                      bias: Optional[torch.Tensor] = None) -> torch.Tensor:
+                      bias: Optional[torch.Tensor] = None, unit_rotated: bool = False,
+                      magnitude: float = 1.0, v_first: Optional[torch.Tensor] = None,
+                      v_lambda: Optional[torch.Tensor] = None) -> torch.Tensor:
     """qkv [T, >= H*D + G*D + Gv*Dv] (q | k | v columns; Gv = v_heads, default
     G; 0: no value columns and none written, for values that are the keys).
-    bias [H*D + G*D] (optional) is added to the q and k columns first.
+    bias [H*D + G*D], or [H*D + G*D + Gv*Dv] with one for the values
+    (optional), is added first.
     RMS norm of every query and key head over its D channels with the float32
     weights [D] (shared by heads; both None: no norm), then rotation of the
-    channel pairs (2i, 2i+1), i < len(inv_freq), by position * inv_freq[i] —
-    all in float32; k and v are written to their pages; returns q [T, H, D]."""
+    channel pairs (2i, 2i+1), i < len(inv_freq), by position * inv_freq[i],
+    cos and sin times `magnitude`. unit_rotated (with no norm weights): after the
+    rotation heads are divided by their root mean square. v_first (another
+    layer's value cache, same shape) with v_lambda (float32 [1]): v becomes
+    (1 - v_lambda) v + v_lambda * v_first's row of the token. All in float32;
+    k and v are written to their pages; returns q [T, H, D]."""
     T = qkv.shape[0]
     Gv = G if v_heads is None else v_heads
-    assert bias is None or (bias.dtype == qkv.dtype and bias.numel() == (H + G) * D)
+    n_qk, n_v = (H + G) * D, Gv * Dv
+    assert bias is None or (bias.dtype == qkv.dtype and bias.is_contiguous()
+                            and bias.numel() in (n_qk, n_qk + n_v))
+    assert not (unit_rotated and q_norm_w is not None)
+    assert (v_first is None) == (v_lambda is None)
+    if v_first is not None:
+        assert v_first.shape == v_cache.shape and v_first.dtype == v_cache.dtype and Gv > 0
+        assert v_lambda.dtype == torch.float32 and v_lambda.numel() == 1
     assert 2 * inv_freq.numel() <= D and (q_norm_w is None) == (k_norm_w is None)
     if not qkv.is_cuda:
         return torch_ref.attn_rope_prepare(qkv, q_norm_w, k_norm_w, inv_freq, H, G, D, Dv, eps,
                                            k_cache, v_cache, _positions(sb), sb.slot_mapping,
-                                           Gv, bias)
+                                           Gv, bias, unit_rotated, magnitude, v_first, v_lambda)
     lib, hip = _lib()
     assert k_cache.dtype == qkv.dtype and v_cache.dtype == qkv.dtype
     assert k_cache.shape[2:] == (G, D) and (Gv == 0 or v_cache.shape[2:] == (Gv, Dv))
@@ -441,6 +490,8 @@ def attn_rope_prepare(qkv: torch.Tensor, q_norm_w: Optional[torch.Tensor],
     for t in (q_norm_w, k_norm_w, inv_freq):
         assert t is None or (t.dtype == torch.float32 and t.is_contiguous())
     assert q_norm_w is None or (q_norm_w.numel() == D and k_norm_w.numel() == D)
+    assert v_first is None or v_first.is_contiguous()
+    vbias = bias[n_qk:] if bias is not None and bias.numel() > n_qk else None
     q = torch.empty(T, H, D, dtype=qkv.dtype, device=qkv.device)
     rc = lib.oa_attn_rope_prepare(
         hip.current_stream_ptr(), qkv.data_ptr(), _rows(qkv),
@@ -450,7 +501,9 @@ def attn_rope_prepare(qkv: torch.Tensor, q_norm_w: Optional[torch.Tensor],
         inv_freq.data_ptr(), inv_freq.numel(), q.data_ptr(),
         k_cache.data_ptr(), v_cache.data_ptr(), sb.slot_mapping.data_ptr(),
         sb.seq_of_t.data_ptr(), sb.cu_t.data_ptr(), sb.past_t.data_ptr(), sb.num_seqs, T,
-        H, G, Gv, D, Dv, eps, _dt(qkv))
+        H, G, Gv, D, Dv, eps, _dt(qkv), vbias.data_ptr() if vbias is not None else None,
+        int(unit_rotated), float(magnitude), v_first.data_ptr() if v_first is not None else None,
+        v_lambda.data_ptr() if v_lambda is not None else None)
     hip.check(rc, "oa_attn_rope_prepare")
     return q
 
@@ -632,6 +685,36 @@ def add_layer_norm(residual: torch.Tensor, w: Optional[torch.Tensor], eps: float
         out.data_ptr() if out is not None else None, _dt(out) if out is not None else 1,
         T, C, float(eps))
     hip.check(rc, "oa_add_layer_norm")
+    return out
+
+
+def add_rms_norm(residual: torch.Tensor, w: Optional[torch.Tensor], eps: float, out_dtype,
+                 y: Optional[torch.Tensor] = None, offset: float = 0.0) -> Optional[torch.Tensor]:
+    """One launch for the add after a layer and the RMS norms of the next:
+    residual (float32 [T, C], in place) += y ([T, C], or partial planes
+    [n, T, C] that add up, linear_partials). With w (float32 [P, C]): returns
+    [P, T, C] in out_dtype, plane p the new residual divided by
+    sqrt(mean(x^2) + eps), times offset + w[p]; float32 inside."""
+    T, C = residual.shape
+    assert residual.dtype == torch.float32 and residual.is_contiguous()
+    assert w is None or (w.dtype == torch.float32 and w.dim() == 2 and w.shape[1] == C
+                         and w.is_contiguous())
+    if not residual.is_cuda:
+        return torch_ref.add_rms_norm(residual, y, w, eps, out_dtype, offset)
+    lib, hip = _lib()
+    P = 0 if w is None else w.shape[0]
+    out = torch.empty(P, T, C, dtype=out_dtype, device=residual.device) if P else None
+    ny, yp, rows = 1, 0, 0
+    if y is not None:
+        if y.dim() == 3:
+            ny, yp = y.shape[0], y.stride(0)
+        rows = _rows(y[0] if y.dim() == 3 else y)
+        assert y.shape[-2:] == (T, C)
+    rc = lib.oa_add_rms_norm(
+        hip.current_stream_ptr(), residual.data_ptr(), y.data_ptr() if y is not None else None,
+        rows, ny, yp, _dt(y) if y is not None else 1, w.data_ptr() if w is not None else None, P,
+        float(offset), out.data_ptr() if P else None, T * C, _dt(out) if P else 1, T, C, float(eps))
+    hip.check(rc, "oa_add_rms_norm")
     return out
 
 
@@ -973,6 +1056,25 @@ def act_rows(x: torch.Tensor, act: str = "relu2",
     return out
 
 
+def act_pair_rows(x: torch.Tensor, act: str = "silu",
+                  out: Optional[torch.Tensor] = None) -> torch.Tensor:
+    """Gated activation on rows of alternating gate and up columns: x [T, 2I]
+    (may be a column slice, and so may `out`) -> act(x[:, 2i]) * x[:, 2i + 1],
+    [T, I]; act "silu" or "gelu_tanh", float32 inside."""
+    T, n = x.shape
+    assert n % 2 == 0 and act in ("silu", "gelu_tanh")
+    if not x.is_cuda:
+        y = torch_ref.act_pair_rows(x, act)
+        return y if out is None else out.copy_(y)
+    lib, hip = _lib()
+    if out is None:
+        out = torch.empty(T, n // 2, dtype=x.dtype, device=x.device)
+    assert out.shape == (T, n // 2) and out.dtype == x.dtype
+    hip.check(lib.oa_act_pair_rows(hip.current_stream_ptr(), x.data_ptr(), _rows(x), out.data_ptr(),
+                                   _rows(out), T, n // 2, _dt(x), ACTS[act]), "oa_act_pair_rows")
+    return out
+
+
 def moe_pairs_plain(x: torch.Tensor, w1: torch.Tensor, w2: torch.Tensor, idx: torch.Tensor,
                     wts: torch.Tensor, act: str = "relu2") -> torch.Tensor:
     """Routed ungated experts for few tokens, two launches, no host sync:
@@ -1044,12 +1146,19 @@ def lowrank_decay(a1: torch.Tensor, w2: torch.Tensor, w0: torch.Tensor) -> torch
 class RowGroup:
     """Rows [begin, end) of a grouped projection weight (both multiples of
     16): they read plane `plane` of the stacked inputs; act: None | "silu" |
-    "gelu_tanh" applied to the result."""
+    "gelu_tanh" applied to the result. paired (with an act): gate and up rows
+    alternate, the result is act(gate) * up."""
 
     begin: int
     end: int
     plane: int = 0
     act: Optional[str] = None
+    paired: bool = False
+
+    @property
+    def width(self) -> int:
+        """Columns of the result."""
+        return (self.end - self.begin) // (2 if self.paired else 1)
 
 
 # columns of K a block of the split product takes
@@ -1083,7 +1192,7 @@ def grouped_linear(x: torch.Tensor, w: torch.Tensor, groups: List[RowGroup],
                    outs: Optional[List[Optional[torch.Tensor]]] = None) -> List[torch.Tensor]:
     """All projections of a layer at once: x [P, T, K] stacked inputs, w [N, K]
     cut into row groups that cover it in order; group g's result is
-    act(x[plane] @ w[begin:end]^T), [T, end - begin], written to outs[g] (may
+    act(x[plane] @ w[begin:end]^T), [T, width], written to outs[g] (may
     be a column slice) where given. Decode-sized bf16 steps are one launch
     with the activation in its epilogue; larger ones run one library GEMM per
     run of groups that read the same plane."""
@@ -1100,11 +1209,11 @@ def grouped_linear(x: torch.Tensor, w: torch.Tensor, groups: List[RowGroup],
         from opsagent_amd.ops import hip_lib as hip
 
         assert x.is_contiguous() and w.is_contiguous() and w.dtype == x.dtype
-        width = sum(g.end - g.begin for g, o in zip(groups, outs) if o is None)
+        width = sum(g.width for g, o in zip(groups, outs) if o is None)
         buf = torch.empty(T, width, dtype=x.dtype, device=x.device) if width else None
         at = 0
         for i, g in enumerate(groups):
-            n = g.end - g.begin
+            n = g.width
             if outs[i] is None:
                 outs[i] = buf[:, at : at + n]
                 at += n
@@ -1115,7 +1224,7 @@ def grouped_linear(x: torch.Tensor, w: torch.Tensor, groups: List[RowGroup],
             hip.current_stream_ptr(), x.data_ptr(), w.data_ptr(), T, N, K, n,
             (ctypes.c_int * n)(*[g.end for g in groups]),
             (ctypes.c_int * n)(*[g.plane for g in groups]),
-            (ctypes.c_int * n)(*[code[g.act] for g in groups]),
+            (ctypes.c_int * n)(*[code[g.act] + (4 if g.paired else 0) for g in groups]),
             (ctypes.c_void_p * n)(*[o.data_ptr() for o in outs]),
             (ctypes.c_int64 * n)(*[_rows(o) for o in outs]), int(mfma))
         hip.check(rc, "oa_gemv_grouped")
@@ -1130,7 +1239,9 @@ def grouped_linear(x: torch.Tensor, w: torch.Tensor, groups: List[RowGroup],
         for k in range(i, j + 1):
             g = groups[k]
             part = y[:, g.begin - lo : g.end - lo]
-            if g.act is not None:
+            if g.paired:
+                outs[k] = act_pair_rows(part, g.act, out=outs[k])
+            elif g.act is not None:
                 outs[k] = act_rows(part, g.act, out=outs[k])
             elif outs[k] is not None:
                 outs[k].copy_(part)

@@ -363,17 +363,22 @@ def dyt_norm(y, post, residual, nxt, out_dtype, bias=None, extra=None):
 
 
 def attn_rope_prepare(qkv, q_norm_w, k_norm_w, inv_freq, H, G, D, Dv, eps, k_cache, v_cache,
-                      positions, slot_mapping, v_heads=None, bias=None):
+                      positions, slot_mapping, v_heads=None, bias=None, unit_rotated=False,
+                      magnitude=1.0, v_first=None, v_lambda=None):
     """Per-head RMS norm of q and k (weight [D] shared by heads; None: no
     norm), then rotation of channel pairs (2i, 2i+1), i < len(inv_freq), by
     position * inv_freq[i]; k and v (v_heads heads, default G; 0: no value
     columns, none written) go to their cache slots, q is returned [T, H, D].
-    bias [H*D + G*D] is added to the q and k columns first."""
+    bias [H*D + G*D], or over the v columns too, is added first. unit_rotated:
+    heads are divided by their root mean square after the rotation instead.
+    magnitude multiplies cos and sin. v_first (a value cache) with v_lambda:
+    v <- (1 - v_lambda) v + v_lambda * the token's row of v_first."""
     T = qkv.shape[0]
     Gv = G if v_heads is None else v_heads
     x = qkv[:, : H * D + G * D + Gv * Dv].float()
     if bias is not None:
-        x = torch.cat([x[:, : (H + G) * D] + bias.float(), x[:, (H + G) * D :]], 1)
+        nb_ = bias.numel()
+        x = torch.cat([x[:, :nb_] + bias.float(), x[:, nb_:]], 1)
     q = x[:, : H * D].reshape(T, H, D)
     k = x[:, H * D : H * D + G * D].reshape(T, G, D)
     v = x[:, H * D + G * D :].reshape(T, Gv, Dv)
@@ -383,7 +388,7 @@ def attn_rope_prepare(qkv, q_norm_w, k_norm_w, inv_freq, H, G, D, Dv, eps, k_cac
     r = 2 * inv_freq.numel()
     if r:
         ang = positions.float()[:, None] * inv_freq.float()[None, :]
-        c, s = torch.cos(ang)[:, None, :], torch.sin(ang)[:, None, :]
+        c, s = magnitude * torch.cos(ang)[:, None, :], magnitude * torch.sin(ang)[:, None, :]
 
         def rot(t):
             a, b = t[..., 0:r:2], t[..., 1:r:2]
@@ -393,8 +398,13 @@ def attn_rope_prepare(qkv, q_norm_w, k_norm_w, inv_freq, H, G, D, Dv, eps, k_cac
             return out
 
         q, k = rot(q), rot(k)
+    if unit_rotated:
+        q, k = (t * torch.rsqrt(t.pow(2).mean(-1, keepdim=True) + eps) for t in (q, k))
     nb, bs = k_cache.shape[0], k_cache.shape[1]
     sm = slot_mapping.long()
+    if v_first is not None:
+        lam = v_lambda.float()
+        v = (1.0 - lam) * v + lam * v_first.view(nb * bs, Gv, Dv)[sm].float()
     k_cache.view(nb * bs, G, D)[sm] = k.to(k_cache.dtype)
     if Gv:
         v_cache.view(nb * bs, Gv, Dv)[sm] = v.to(v_cache.dtype)
@@ -402,11 +412,13 @@ def attn_rope_prepare(qkv, q_norm_w, k_norm_w, inv_freq, H, G, D, Dv, eps, k_cac
 
 
 def attention_paged(q, k_cache, v_cache, cu, past, block_table, scale, slopes=None,
-                    gate_logits=None, window=None, sinks=None, softcap=None):
+                    gate_logits=None, window=None, sinks=None, softcap=None, keep_first=0,
+                    gate_channels=False):
     """Causal softmax attention of each new token over its sequence's cached
     keys. Options: a linear distance penalty slope_h*(i-j), a window (key j
-    seen iff i - j < window), a per-head sink term exp(sink_h) in the
-    denominator, a sigmoid gate on each head's output, a soft cap
+    seen iff i - j < window or j < keep_first), a per-head sink term exp(sink_h)
+    in the denominator, a sigmoid gate on each head's output (gate_channels: on
+    each of its channels), a soft cap
     cap * tanh(score / cap) on the scaled score. The cache may hold fewer
     value heads than key heads: key head g reads value head g mod Gv."""
     T, H, D = q.shape
@@ -419,7 +431,7 @@ def attention_paged(q, k_cache, v_cache, cu, past, block_table, scale, slopes=No
         if hi == lo:
             continue
         total = past[b] + hi - lo
-        first = max(0, past[b] - window + 1) if window else 0
+        first = max(0, past[b] - window + 1) if window and not keep_first else 0
         fb = first // bs
         first = fb * bs
         nblk = (total + bs - 1) // bs
@@ -440,7 +452,7 @@ def attention_paged(q, k_cache, v_cache, cu, past, block_table, scale, slopes=No
             s = s - slopes.float().view(H, 1, 1) * (i - j)
         hide = j > i
         if window:
-            hide = hide | (i - j >= window)
+            hide = hide | ((i - j >= window) & (j >= keep_first))
         s = s.masked_fill(hide, float("-inf"))
         if sinks is not None:
             s = torch.cat([s, sinks.float().view(H, 1, 1).expand(H, s.shape[1], 1)], -1)
@@ -449,7 +461,8 @@ def attention_paged(q, k_cache, v_cache, cu, past, block_table, scale, slopes=No
             p = p[..., :-1]
         o = torch.einsum("hij,jhd->ihd", p, vv)
         if gate_logits is not None:
-            o = o * torch.sigmoid(gate_logits[lo:hi].float()).unsqueeze(-1)
+            g = torch.sigmoid(gate_logits[lo:hi].float())
+            o = o * (g.reshape(hi - lo, H, Dv) if gate_channels else g.unsqueeze(-1))
         out[lo:hi] = o.to(q.dtype)
     return out.view(T, H * Dv)
 
@@ -531,6 +544,26 @@ def add_layer_norm(residual, y, w, eps, out_dtype, y2=None, y2_gate=None):
     mu = residual.mean(-1, keepdim=True)
     d = residual - mu
     return (d * torch.rsqrt(d.pow(2).mean(-1, keepdim=True) + eps) * w.float()).to(out_dtype)
+
+
+def add_rms_norm(residual, y, w, eps, out_dtype, offset=0.0):
+    """residual (float32 [T, C], in place) += y ([T, C], or planes [n, T, C]
+    that add up). With w [P, C]: returns [P, T, C], the new residual divided
+    by sqrt(mean(x^2) + eps), times offset + w[p]."""
+    if y is not None:
+        residual += y.float().sum(0) if y.dim() == 3 else y.float()
+    if w is None:
+        return None
+    n = residual * torch.rsqrt(residual.pow(2).mean(-1, keepdim=True) + eps)
+    return torch.stack([n * (offset + w[p].float()) for p in range(w.shape[0])]).to(out_dtype)
+
+
+def act_pair_rows(x, act):
+    """x [T, 2I] of alternating gate and up columns: act(gate) * up, [T, I]."""
+    z = x.float()
+    g, u = z[:, 0::2], z[:, 1::2]
+    a = torch.nn.functional.silu(g) if act == "silu" else gelu_tanh(g)
+    return (a * u).to(x.dtype)
 
 
 def _rotate_pairs(x, pos, inv_freq):

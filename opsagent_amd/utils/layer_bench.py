@@ -24,6 +24,8 @@ from opsagent_amd.engine.config import (
     rafodra_spec_from_dict,
     rimonex_config_dict,
     rimonex_spec_from_dict,
+    safesun_config_dict,
+    safesun_spec_from_dict,
     suzulix_config_dict,
     suzulix_spec_from_dict,
     vazilorn_config_dict,
@@ -106,7 +108,19 @@ def specs_for(size) -> Dict[str, object]:
             name=f"rimonex-{tag}-{name}",
         )
 
+    def ss(window, tag):
+        # both kinds of gated rotary attention (keys of the first four tokens
+        # stay in sight), values mixed with the first layer's: heads and gated
+        # feed-forwards of llama's sizes
+        return safesun_spec_from_dict(
+            safesun_config_dict(vocab=32000, width=width, pattern=("AdBdBdAd" * layers)[:2 * layers],
+                                heads=heads, kv_heads=kv, dim=dim, vdim=dim, window=window,
+                                keep_first=4, rot_base=500000.0, ff=ff),
+            name=f"safesun-{tag}-{name}",
+        )
+
     return {
+        "safesun": ss(8192, "dense"), "safesun-w512": ss(512, "w512"),
         "rimonex": rx("PdDd", 8192, "dense"), "rimonex-w512": rx("PdDd", 512, "w512"),
         "suzulix": sz("LmAmRmRm", 2, "moe"),
         # mixers alone (no feed-forward) beside Rafodra's: what the streams,
@@ -125,6 +139,7 @@ def specs_for(size) -> Dict[str, object]:
 # which model each one is measured against
 BASELINE_OF = {"povazen": "llama", "vazilorn": "llama", "vazilorn-w512": "llama",
                "vazilorn-moe": "llama-moe", "rafodra": "povazen", "rafodra-moe": "vazilorn-moe",
+               "safesun": "vazilorn", "safesun-w512": "vazilorn-w512",
                "rimonex": "povazen", "rimonex-w512": "rimonex",
                "suzulix": "rafodra-moe", "suzulix-mix": "rafodra-mix"}
 

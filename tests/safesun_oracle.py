@@ -85,15 +85,10 @@ def rotate(x, rot, first=0):
         return x
     half = rot["dims"] // 2
     f, m = frequencies(rot)
-    out = x.clone()
-    for t in range(x.shape[0]):
-        for i in range(half):
-            a = (first + t) * f[i]
-            c, s = m * math.cos(a), m * math.sin(a)
-            u, v = x[t, :, i], x[t, :, i + half]
-            out[t, :, i] = u * c - v * s
-            out[t, :, i + half] = v * c + u * s
-    return out
+    a = torch.arange(first, first + x.shape[0], dtype=F64)[:, None] * torch.tensor(f, dtype=F64)
+    c, s = m * torch.cos(a)[:, None, :], m * torch.sin(a)[:, None, :]
+    u, v = x[..., :half], x[..., half:2 * half]
+    return torch.cat([u * c - v * s, v * c + u * s, x[..., 2 * half:]], -1)
 
 
 def sees(i, j, mask):
@@ -107,19 +102,17 @@ def sees(i, j, mask):
 def heads_softmax(q, k, v, scale, mask, plus_one, past=0):
     """q [n, H, D] at positions past .., k [past + n, G, D], v [.., G, Dv]."""
     n, H, _ = q.shape
-    G = k.shape[1]
+    G, total = k.shape[1], past + q.shape[0]
+    hidden = torch.tensor([[not sees(past + r, j, mask) for j in range(total)] for r in range(n)])
     out = torch.zeros(n, H, v.shape[-1], dtype=F64)
-    for r in range(n):
-        i = past + r
-        seen = [j for j in range(i + 1) if sees(i, j, mask)]
-        for hh in range(H):
-            g = hh // (H // G)
-            s = (k[seen, g] @ q[r, hh]) * scale
-            top = s.max()
-            z = torch.exp(s - top).sum()
-            if plus_one:
-                z = z + torch.exp(-top)
-            out[r, hh] = (torch.exp(s - top) / z) @ v[seen, g]
+    for hh in range(H):
+        g = hh // (H // G)
+        s = ((q[:, hh] @ k[:, g].T) * scale).masked_fill(hidden, -math.inf)
+        top = s.max(1, keepdim=True).values
+        z = torch.exp(s - top).sum(1, keepdim=True)
+        if plus_one:
+            z = z + torch.exp(-top)
+        out[:, hh] = (torch.exp(s - top) / z) @ v[:, g]
     return out
 
 

@@ -62,5 +62,6 @@ def test_mixers_library_exports():
               "oa_moe_pairs_gateup", "oa_moe_pairs_down", "oa_add_layer_norm",
               "oa_latent_kv_prepare", "oa_latent_q_assemble", "oa_decay_scan",
               "oa_gated_rms_norm", "oa_hyper_norm", "oa_rope_rows", "oa_combine_norm_gate",
-              "oa_act_rows", "oa_moe_pairs_up", "oa_shift_mix", "oa_lowrank_decay"]:
+              "oa_act_rows", "oa_moe_pairs_up", "oa_shift_mix", "oa_lowrank_decay",
+              "oa_add_rms_norm", "oa_act_pair_rows"]:
         assert hasattr(lib, s), f"missing {s}"

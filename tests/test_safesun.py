@@ -1,0 +1,972 @@
+"""The Safesun decoder in the framework (engine, paged cache, scheduler,
+ops/kernels) against the plain oracle in safesun_oracle.py.
+
+Unmarked cases run on the CPU path (float32); gpu-marked cases run the HIP
+kernels in float32 and bfloat16. Configurations are small and irregular:
+sizes that are not powers of two, key size != value size, fewer kv heads than
+heads, windows that are neither page nor tile multiples, layers without a
+feed-forward, layers without value mixing before, between and after those
+with it.
+"""
+
+import copy
+import json
+
+import pytest
+import torch
+
+import safesun_oracle as O
+from opsagent_amd.engine.config import (
+    apply_tensor_shapes,
+    get_model_spec,
+    safesun_config_dict,
+    safesun_spec_from_dict,
+)
+from opsagent_amd.engine.engine import LLMEngine, SamplingParams
+from opsagent_amd.engine.replay import TraceReplayer
+from opsagent_amd.ops import mixer_ops as mx
+
+gpu = pytest.mark.gpu
+MODES = [
+    pytest.param(("cpu", "fp32"), id="cpu-f32"),
+    pytest.param(("cuda", "fp32"), id="gpu-f32", marks=gpu),
+    pytest.param(("cuda", "bf16"), id="gpu-bf16", marks=gpu),
+]
+F64 = torch.float64
+YARN = {"factor": 3.0, "fast": 12.0, "slow": 1.5, "original": 60}
+
+
+def _skip_if_wrong_device(device):
+    if device == "cpu" and torch.cuda.is_available():
+        pytest.skip("the engine picks the GPU on this box; CPU path is covered on CPU runs")
+
+
+def tdtype(name):
+    return torch.float32 if name == "fp32" else torch.bfloat16
+
+
+def dev_of(device):
+    return "cuda" if device == "cuda" else "cpu"
+
+
+def close(got, want, dtype, what="", loose=1.0):
+    got, want = got.detach().double().cpu(), want.detach().double().cpu()
+    assert got.shape == want.shape, (got.shape, want.shape)
+    err = (got - want).pow(2).mean().sqrt() / (want.pow(2).mean().sqrt() + 1e-9)
+    worst = (got - want).abs().max() / (want.abs().max() + 1e-9)
+    if dtype == "fp32":
+        assert err < 3e-5 * loose and worst < 3e-4 * loose, f"{what}: rel rms {err:.3e}, worst {worst:.3e}"
+    else:
+        assert err < 1e-2 * loose and worst < 5e-2 * loose, f"{what}: rel rms {err:.3e}, worst {worst:.3e}"
+
+
+def _bf16_nearest(x):
+    return x.to(torch.bfloat16).double()
+
+
+def _bf16_chop(x):
+    """Rounding toward zero: another realisation of the same noise level."""
+    f = x.float()
+    return (f.view(torch.int32) & -65536).view(torch.float32).double()
+
+
+def oracle_runs(cfg, W, toks, dtype):
+    """The oracle's logits and residuals after every layer, and in bf16 mode
+    the same from runs whose low-precision points are rounded to bfloat16 in
+    two ways: how far rounding alone moves each position."""
+    layers, noisy = [], []
+    exact = O.forward(cfg, W, toks, layers)
+    if dtype == "bf16":
+        for fn in (_bf16_nearest, _bf16_chop):
+            with O.rounding(fn):
+                ls = []
+                lg = O.forward(cfg, W, toks, ls)
+            noisy.append((lg, ls))
+    return exact, layers, noisy
+
+
+def close_rows(got, want, noisy, dtype, what=""):
+    """Row by row (a row is a position). float32: the strict bounds of close().
+    bfloat16: a row may be as far from the oracle as 1e-2 of its size plus
+    three times what rounding alone moved it in the oracle's own rounded runs."""
+    if dtype == "fp32":
+        return close(got, want, dtype, what)
+    got, want = got.detach().double().cpu(), want.detach().double().cpu()
+    assert got.shape == want.shape, (got.shape, want.shape)
+    size = want.pow(2).mean(-1).sqrt() + 1e-9
+    err = (got - want).pow(2).mean(-1).sqrt() / size
+    moved = torch.stack([(n.double() - want).pow(2).mean(-1).sqrt() / size for n in noisy]).max(0).values
+    bad = (err > 1e-2 + 3.0 * moved).nonzero().flatten().tolist()
+    assert not bad, f"{what}: rows {bad[:8]}: err {err[bad[:8]].tolist()}, rounding alone {moved[bad[:8]].tolist()}"
+
+
+def rounded(W, dtype):
+    """The weights the engine holds."""
+    return W if dtype != "bf16" else {k: v.to(torch.bfloat16).float() for k, v in W.items()}
+
+
+def model_close(got, cfg, W, toks, dtype, what=""):
+    exact, _, noisy = oracle_runs(cfg, rounded(W, dtype), toks, dtype)
+    close_rows(got, exact, [lg for lg, _ in noisy], dtype, what)
+
+
+def make_cfg(pattern="adBdA-bdAdBd", width=42, vocab=97, **kw):
+    base = dict(heads=6, kv_heads=2, dim=12, vdim=10, window=21, keep_first=3, scale=0.4, rot_dims=8,
+                rot_base=3000.0, rot_scaling=YARN, heads_2=4, dim_2=14, window_2=13, keep_first_2=5,
+                scale_2=1.1, rot_dims_2=14, rot_base_2=700.0, ff=52, eps=1e-5)
+    base.update(kw)
+    return safesun_config_dict(vocab, width, pattern, **base)
+
+
+def x16_cfg(pattern="BdA-bdAdBd", **kw):
+    """Sizes the matrix-core attention kernel and the vector paths take."""
+    base = dict(width=80, heads=4, kv_heads=2, dim=32, vdim=48, rot_dims=32, heads_2=8, dim_2=16,
+                rot_dims_2=12, ff=96)
+    base.update(kw)
+    return make_cfg(pattern, **base)
+
+
+def build_engine(cfg, W, dtype="fp32", blocks=64, block_size=8, slots=4, **extra):
+    spec = apply_tensor_shapes(safesun_spec_from_dict(cfg), {k: tuple(v.shape) for k, v in W.items()})
+    eng = LLMEngine(dict({
+        "model": spec, "dtype": dtype, "kv_num_blocks": blocks,
+        "kv_block_size": block_size, "max_batch_size": slots, "state_slots": slots,
+        "tokenizer_check": False, "max_seq_len": 4096, "max_prefill_chunk": 4096,
+    }, **extra))
+    eng.model.load_named_tensors(rounded(W, dtype))
+    return eng
+
+
+def tokens_for(cfg, n, seed):
+    g = torch.Generator().manual_seed(seed)
+    return torch.randint(0, cfg["vocab"], (n,), generator=g).tolist()
+
+
+def replay(eng, schedule):
+    """schedule: list of steps; step = list of (id, tokens, last?) -> id -> logits of every position."""
+    rp = TraceReplayer(eng)
+    got = {}
+    for step in schedule:
+        entries = [{"id": i, "tokens": t, "want": list(range(len(t)))} for i, t, _ in step]
+        end = [i for i, _, last in step if last]
+        out = rp.step(entries, end)
+        off = 0
+        for i, t, _ in step:
+            got.setdefault(i, []).append(out[off:off + len(t)])
+            off += len(t)
+    return {i: torch.cat(v, 0) for i, v in got.items()}
+
+
+def cut(tokens, sizes):
+    out, at, k = [], 0, 0
+    while at < len(tokens):
+        n = sizes[k % len(sizes)]
+        out.append(tokens[at:at + n])
+        at += n
+        k += 1
+    return out
+
+
+def serve(eng, toks, sizes):
+    parts = cut(toks, sizes)
+    return replay(eng, [[("a", p, k == len(parts) - 1)] for k, p in enumerate(parts)])["a"]
+
+
+# --------------------------------------------------------------------------
+# mechanisms alone
+
+
+@pytest.mark.parametrize("dims,base,sc", [
+    (64, 20000.0, dict(factor=2.5, fast=32.0, slow=1.0, original=4096)),
+    (16, 500.0, dict(factor=40.0, fast=4.0, slow=2.0, original=100)),
+    (12, 10000.0, dict(factor=1.0, fast=32.0, slow=1.0, original=64)),
+    (10, 10000.0, dict(factor=4.0, fast=1e9, slow=1e8, original=64)),       # both ends clamp to 0
+    (10, 1.5, dict(factor=4.0, fast=1e-9, slow=1e-9, original=64)),         # all pairs kept
+    (8, 50000.0, dict(factor=7.0, fast=3.0, slow=3.0, original=256)),       # a step or one index
+    (2, 100.0, None), (36, 1e6, None),
+])
+def test_rotation_frequencies(dims, base, sc):
+    want, mag = O.frequencies({"dims": dims, "base": base, "scaling": sc})
+    got = mx.rotary_inv_freq(dims, base, sc)
+    assert got.dtype == torch.float32 and got.numel() == dims // 2
+    assert (got.double() / torch.tensor(want, dtype=F64) - 1.0).abs().max() < 1e-7
+    assert abs(mx.rotary_magnitude(sc) - mag) < 1e-12
+    if sc and sc["factor"] > 1.0 and 1e-6 < sc["fast"] < 1e6:
+        plain = mx.rotary_inv_freq(dims, base)
+        assert not torch.equal(got, plain) and mag > 1.0
+
+
+PREP_GEOMS = [(6, 2, 12, 10, 8), (4, 2, 32, 16, 32), (3, 1, 7, 5, 6), (2, 2, 136, 24, 40),
+              (8, 8, 64, 64, 0), (1, 1, 2, 1, 2), (5, 1, 16, 8, 4)]
+
+
+@pytest.mark.parametrize("mode", MODES)
+@pytest.mark.parametrize("second", [False, True])
+@pytest.mark.parametrize("H,G,D,Dv,R", PREP_GEOMS)
+def test_query_key_value_preparation(mode, second, H, G, D, Dv, R):
+    """Projection columns to queries and cached rows for two sequences, one far
+    out: weighted norm then rotation with a magnitude, or biases, rotation,
+    unit norm; values mixed with another layer's cached row of the same token.
+    Only the slots of the new tokens are written."""
+    device, dtype = mode
+    _skip_if_wrong_device(device)
+    dev, dt = dev_of(device), tdtype(dtype)
+    g = torch.Generator().manual_seed(H * D + Dv)
+    rn = lambda *s: torch.randn(*s, generator=g)   # noqa: E731
+    eps, mag, lam, T = 0.02, 1.25, 0.3, 5
+    n = (H + G) * D + G * Dv
+    x = rn(T, n + 8).to(dt)[:, :n]
+    b = rn(n).to(dt) if second else None
+    qw, kw = (None, None) if second else (1.0 + 0.2 * rn(D), 1.0 + 0.2 * rn(D))
+    freq = mx.rotary_inv_freq(R, 50.0)
+    first = rn(7, 8, G, Dv).to(dt)
+    kc, vc = torch.zeros(7, 8, G, D, dtype=dt), torch.zeros(7, 8, G, Dv, dtype=dt)
+    kc, vc, first_d = kc.to(dev), vc.to(dev), first.to(dev)
+    sb = mx.SeqBatch.build([(14, 3, 0, [6, 2, 4]), (0, 2, 1, [1])], 8, dev)
+    d = lambda t: None if t is None else t.to(dev)   # noqa: E731
+    q = mx.attn_rope_prepare(x.to(dev), d(qw), d(kw), freq.to(dev), H, G, D, Dv, eps, kc, vc, sb,
+                             bias=d(b), unit_rotated=second, magnitude=mag, v_first=first_d,
+                             v_lambda=torch.tensor([lam]).to(dev))
+    y = x.double() + (b.double() if second else 0.0)
+    heads = y[:, : (H + G) * D].reshape(T, H + G, D)
+    pos = torch.tensor([14, 15, 16, 0, 1], dtype=F64)
+
+    def turn(z):
+        a = pos[:, None, None] * freq.double()
+        c, s = mag * torch.cos(a), mag * torch.sin(a)
+        out = z.clone()
+        u, v = z[..., 0:R:2], z[..., 1:R:2]
+        out[..., 0:R:2], out[..., 1:R:2] = u * c - v * s, v * c + u * s
+        return out
+
+    if second:
+        heads = O.unit_rms(turn(heads), eps)
+    else:
+        w = torch.cat([qw.expand(H, D), kw.expand(G, D)]).double()
+        heads = turn(O.unit_rms(heads, eps) * w)
+    where = [(2, 6), (2, 7), (4, 0), (1, 0), (1, 1)]
+    rows = lambda c: torch.stack([c[i, j] for i, j in where]).double().cpu()   # noqa: E731
+    v = (1 - lam) * y[:, (H + G) * D:].reshape(T, G, Dv) + lam * rows(first)
+    close(q, heads[:, :H], dtype, "queries", loose=0.4 if dtype == "bf16" else 1.0)
+    close(rows(kc), heads[:, H:], dtype, "keys", loose=0.4 if dtype == "bf16" else 1.0)
+    close(rows(vc), v, dtype, "values", loose=0.4 if dtype == "bf16" else 1.0)
+    assert int((kc != 0).flatten(2).any(-1).sum()) == 5 and int((vc != 0).flatten(2).any(-1).sum()) == 5
+    assert torch.equal(first_d.cpu(), first)
+
+
+@pytest.mark.parametrize("mode", MODES)
+@pytest.mark.parametrize("second", [False, True])
+def test_values_without_mixing_or_bias_pass_unchanged(mode, second):
+    device, dtype = mode
+    _skip_if_wrong_device(device)
+    dev, dt = dev_of(device), tdtype(dtype)
+    H, G, D, Dv = (4, 2, 16, 8) if second else (3, 1, 6, 5)
+    x = torch.randn(4, (H + G) * D + G * Dv, generator=torch.Generator().manual_seed(1)).to(dt)
+    kc, vc = torch.zeros(1, 8, G, D, dtype=dt, device=dev), torch.zeros(1, 8, G, Dv, dtype=dt, device=dev)
+    sb = mx.SeqBatch.build([(0, 4, 0, [0])], 8, dev)
+    mx.attn_rope_prepare(x.to(dev), None, None, torch.empty(0, device=dev), H, G, D, Dv, 1e-5, kc, vc, sb,
+                         unit_rotated=True)
+    assert torch.equal(vc[0, :4].reshape(4, -1).cpu(), x[:, (H + G) * D:])
+
+
+def _attend(mode, q, k, v, past, scale, mask, plus_one, gate=None, block_size=8):
+    """attention_paged for ONE sequence whose cache rows are given whole
+    (k [total, G, D], v [total, G, Dv]); q [n, H, D] at positions past ...
+    The result goes to columns of a wider buffer."""
+    device, dtype = mode
+    dev, dt = dev_of(device), tdtype(dtype)
+    (n, H, D), (total, G, Dv) = q.shape, v.shape
+    nblk = (total + block_size - 1) // block_size
+    order = list(range(nblk + 2, 2, -1))                    # pages in falling order
+    kc = torch.full((nblk + 4, block_size, G, D), 50.0, dtype=dt)
+    vc = torch.full((nblk + 4, block_size, G, Dv), 50.0, dtype=dt)
+    for j in range(total):
+        kc[order[j // block_size], j % block_size] = k[j].to(dt)
+        vc[order[j // block_size], j % block_size] = v[j].to(dt)
+    sb = mx.SeqBatch.build([(past, n, 0, order)], block_size, dev)
+    wide = torch.full((n, H * Dv + 32), 7.0, dtype=dt, device=dev)
+    gl = None
+    if gate is not None:
+        gl = torch.cat([gate, gate], 1).to(dt).to(dev)[:, : H * Dv] if Dv % 4 == 0 else gate.to(dt).to(dev)
+    out = mx.attention_paged(q.to(dt).to(dev).contiguous(), kc.to(dev), vc.to(dev), sb, scale,
+                             window=mask.get("size"), keep_first=mask.get("keep_first", 0),
+                             sinks=torch.zeros(H, device=dev) if plus_one else None,
+                             gate_logits=gl, gate_channels=True, out=wide[:, 16:-16])
+    assert bool((wide[:, :16] == 7.0).all()) and bool((wide[:, -16:] == 7.0).all())
+    return out.reshape(n, H, Dv).double().cpu()
+
+
+def _attend_reference(dt, q, k, v, past, scale, mask, plus_one, gate=None):
+    f = lambda t: t.to(dt).double()   # noqa: E731
+    o = O.heads_softmax(f(q), f(k), f(v), scale, mask, plus_one, past)
+    return o if gate is None else o * O.sigmoid(f(gate)).reshape(o.shape)
+
+
+WINDOW, KEEP = 72, 70      # neither a multiple of a page nor of a key tile
+
+
+@pytest.mark.parametrize("mode", MODES)
+@pytest.mark.parametrize("plus_one", [False, True])
+@pytest.mark.parametrize("keep", [5, KEEP])
+@pytest.mark.parametrize("target", [0, 1, 4, 5, 7, 8, 63, 64, 69, 70, 71, 150, -1, -8, -64, -71, -72, -73, -74, -80])
+@pytest.mark.parametrize("n", [1, 9, 100])
+def test_one_key_stands_out(mode, plus_one, keep, target, n):
+    """One key (a position, or so many before the end) has a large product
+    with the last query: seen in the window or among the kept first tokens its
+    value dominates the output, otherwise it leaves no trace. For a single
+    decoded token and for portions whose last query is in the first, and in a
+    later, query tile."""
+    device, dtype = mode
+    _skip_if_wrong_device(device)
+    H, G, D, Dv, total = 4, 2, 16, 16, 333
+    past = total - n
+    g = torch.Generator().manual_seed(7)
+    k, v = 0.05 * torch.randn(total, G, D, generator=g), 0.05 * torch.randn(total, G, Dv, generator=g)
+    q = 0.05 * torch.randn(n, H, D, generator=g)
+    at = target if target >= 0 else total + target
+    k[at, :, 0], v[at, :, 1] = 6.0, 4.0
+    q[-1, :, 0] = 6.0
+    mask = {"size": WINDOW, "keep_first": keep}
+    got = _attend(mode, q, k, v, past, 0.5, mask, plus_one)
+    want = _attend_reference(tdtype(dtype), q, k, v, past, 0.5, mask, plus_one)
+    close(got, want, dtype, f"key at {at}")
+    lead = got[-1, :, 1]
+    if total - 1 - at < WINDOW or at < keep:
+        assert bool((lead > 3.9).all()), lead
+    else:
+        assert bool((lead.abs() < 0.2).all()), lead
+
+
+@pytest.mark.parametrize("mode", MODES)
+@pytest.mark.parametrize("n", [1, 100])
+def test_one_is_added_to_the_denominator_once(mode, n):
+    """Zero scores: each of the j visible keys takes 1 / (j + 1). With scores of
+    -4 the one outweighs the keys; without it the weights sum to 1."""
+    device, dtype = mode
+    _skip_if_wrong_device(device)
+    H, G, D, Dv, total = 2, 1, 16, 16, 150
+    k, v = torch.zeros(total, G, D), torch.ones(total, G, Dv)
+    k[..., 0] = -4.0
+    q = torch.zeros(n, H, D)
+    q[:, 1, 0] = 1.0                                        # head 1: every score is -4
+    mask = {"size": 40, "keep_first": 3}
+    got = _attend(mode, q, k, v, total - n, 1.0, mask, True)[..., 0]
+    tol = 1e-5 if dtype == "fp32" else 4e-3
+    seen = torch.tensor([sum(O.sees(total - n + i, j, mask) for j in range(total)) for i in range(n)])
+    assert int(seen[-1]) == 43
+    e4 = torch.exp(torch.tensor(4.0, dtype=F64))
+    assert (got[:, 0] - seen / (seen + 1.0)).abs().max() < tol
+    assert (got[:, 1] - seen / (seen + e4)).abs().max() < tol
+    assert (_attend(mode, q, k, v, total - n, 1.0, mask, False)[..., 0] - 1.0).abs().max() < tol
+
+
+@pytest.mark.parametrize("mode", MODES)
+@pytest.mark.parametrize("score", [-300.0, 300.0])
+def test_extreme_scores_beside_the_one(mode, score):
+    """The added one neither overflows nor vanishes at the ends of the range."""
+    device, dtype = mode
+    _skip_if_wrong_device(device)
+    k, v, q = torch.zeros(20, 1, 16), torch.ones(20, 1, 16), torch.zeros(1, 2, 16)
+    k[..., 0], q[..., 0] = score, 1.0
+    got = _attend(mode, q, k, v, 19, 1.0, {"size": 9, "keep_first": 2}, True)
+    assert bool(torch.isfinite(got).all())
+    assert (got - (1.0 if score > 0 else 0.0)).abs().max() < 1e-5
+
+
+@pytest.mark.parametrize("mode", MODES)
+@pytest.mark.parametrize("H,G,D,Dv", [(6, 2, 12, 10), (4, 2, 32, 48), (3, 1, 7, 5), (32, 1, 16, 16), (5, 5, 64, 16),
+                                      (2, 2, 136, 8), (2, 1, 32, 272), (4, 1, 256, 128), (80, 2, 16, 32)])
+@pytest.mark.parametrize("size,keep", [(21, 3), (None, 0), (1, 1), (8, 64), (30, 0), (2, 200)])
+def test_attention_geometries(mode, H, G, D, Dv, size, keep):
+    device, dtype = mode
+    _skip_if_wrong_device(device)
+    g = torch.Generator().manual_seed(H * D)
+    k, v = torch.randn(90, G, D, generator=g), torch.randn(90, G, Dv, generator=g)
+    mask = {"size": size, "keep_first": keep}
+    for past, n in ((0, 50), (33, 57), (89, 1)):
+        q, gate = torch.randn(n, H, D, generator=g), torch.randn(n, H * Dv, generator=g)
+        args = (q, k[: past + n], v[: past + n], past, 1.5 / D ** 0.5, mask, True, gate)
+        close(_attend(mode, *args), _attend_reference(tdtype(dtype), *args), dtype, f"past {past}, {n} queries")
+
+
+@pytest.mark.parametrize("mode", MODES)
+@pytest.mark.parametrize("D", [12, 32])
+def test_long_context_key_splits(mode, D):
+    """A long context with few queries: key tiles are split over blocks and
+    merged; window, kept tokens, gate and the added one survive the merge."""
+    device, dtype = mode
+    _skip_if_wrong_device(device)
+    g = torch.Generator().manual_seed(D)
+    total, H, G, Dv = 2100, 2, 1, 16
+    k, v = torch.randn(total, G, D, generator=g), torch.randn(total, G, Dv, generator=g)
+    for n in (1, 20):
+        q, gate = torch.randn(n, H, D, generator=g), torch.randn(n, H * Dv, generator=g)
+        for mask in ({"size": 1500, "keep_first": 9}, {"size": 700, "keep_first": 300}, {"size": None}):
+            args = (q, k, v, total - n, 0.4, mask, True, gate)
+            close(_attend(mode, *args), _attend_reference(tdtype(dtype), *args), dtype, f"{n} queries, {mask}")
+
+
+@pytest.mark.parametrize("mode", MODES)
+@pytest.mark.parametrize("T,C", [(1, 40), (5, 7), (3, 192), (2, 4100), (2, 5003), (9, 1)])
+@pytest.mark.parametrize("planes", [1, 2, 3])
+def test_add_and_norms(mode, T, C, planes):
+    """Residual add (plain rows, or partial planes that add up) and several
+    norms of the same row with weights of their own, around zero or around one."""
+    device, dtype = mode
+    _skip_if_wrong_device(device)
+    dev, dt = dev_of(device), tdtype(dtype)
+    g = torch.Generator().manual_seed(T * C + planes)
+    rn = lambda *s: torch.randn(*s, generator=g)   # noqa: E731
+    w, res = 0.3 * rn(planes, C), 3.0 * rn(T, C)
+    for y, offset in ((None, 1.0), (rn(T, C + 4).to(dt)[:, :C], 1.0), (rn(3, T, C), 0.0)):
+        r = res.clone().to(dev)
+        out = mx.add_rms_norm(r, w.to(dev), 0.1, dt, y=None if y is None else y.to(dev), offset=offset)
+        want = res.double()
+        if y is not None:
+            want = want + (y.double() if y.dim() == 2 else y.double().sum(0))
+        close(r, want, "fp32", "residual")
+        assert out.shape == (planes, T, C) and out.dtype == dt
+        for p in range(planes):
+            close(out[p], O.unit_rms(want, 0.1) * (offset + w[p].double()), dtype, f"norm {p}")
+        if y is not None:
+            r = res.clone().to(dev)
+            assert mx.add_rms_norm(r, None, 0.1, dt, y=y.to(dev)) is None
+            close(r, want, "fp32", "add alone")
+    r = res.clone().to(dev)
+    out = mx.add_rms_norm(r, w.to(dev), 1e-6, torch.float32, offset=1.0)     # float32 rows in both modes
+    assert out.dtype == torch.float32 and torch.equal(r.cpu(), res)
+    close(out[0], O.norm(res.double(), w[0].double(), 1e-6), "fp32", "float32 norm")
+
+
+@pytest.mark.parametrize("mode", MODES)
+@pytest.mark.parametrize("act", ["silu", "gelu_tanh"])
+@pytest.mark.parametrize("T,I", [(3, 24), (2, 5), (300, 64), (1, 1), (7, 36)])
+def test_paired_activation(mode, act, T, I):
+    device, dtype = mode
+    _skip_if_wrong_device(device)
+    dev, dt = dev_of(device), tdtype(dtype)
+    g = torch.Generator().manual_seed(T * I)
+    x = (2.0 * torch.randn(T, 2 * I + 16, generator=g)).to(dt)
+    wide = torch.full((T, I + 32), 9.0, dtype=dt, device=dev)
+    got = mx.act_pair_rows(x.to(dev)[:, 8 : 8 + 2 * I], act, out=wide[:, 16 : 16 + I])
+    a, u = x[:, 8 : 8 + 2 * I : 2].double(), x[:, 9 : 9 + 2 * I : 2].double()
+    gelu = lambda z: 0.5 * z * (1.0 + torch.tanh((2.0 / torch.pi) ** 0.5 * (z + 0.044715 * z ** 3)))   # noqa: E731
+    close(got, (O.silu(a) if act == "silu" else gelu(a)) * u, dtype, act)
+    assert bool((wide[:, :16] == 9.0).all()) and bool((wide[:, 16 + I:] == 9.0).all())
+
+
+@pytest.mark.parametrize("mode", MODES)
+@pytest.mark.parametrize("T", [1, 2, 3, 4, 8, 21])
+@pytest.mark.parametrize("K", [24, 40, 1024])
+def test_grouped_projections_with_paired_rows(mode, T, K):
+    """Plain rows from one plane, alternating gate and up rows from another,
+    the activated product in a column slice of a wider buffer."""
+    device, dtype = mode
+    _skip_if_wrong_device(device)
+    dev, dt = dev_of(device), tdtype(dtype)
+    g = torch.Generator().manual_seed(T * K)
+    x = torch.randn(2, T, K, generator=g).to(dt)
+    w = (torch.randn(16 * 9, K, generator=g) * K ** -0.5).to(dt)
+    groups = [mx.RowGroup(0, 32), mx.RowGroup(32, 48), mx.RowGroup(48, 112, 1, "silu", True),
+              mx.RowGroup(112, 144, 1, "gelu_tanh", False)]
+    assert [gr.width for gr in groups] == [32, 16, 32, 32]
+    wide = torch.full((T, 64), 9.0, dtype=dt, device=dev)
+    outs = mx.grouped_linear(x.to(dev), w.to(dev), groups, [None, None, wide[:, 16:48], None])
+    assert outs[2].data_ptr() == wide[:, 16:48].data_ptr()
+    for gr, o in zip(groups, outs):
+        want = x[gr.plane].double() @ w[gr.begin:gr.end].double().T
+        if gr.paired:
+            want = O.silu(want[:, 0::2]) * want[:, 1::2]
+        elif gr.act:
+            want = 0.5 * want * (1.0 + torch.tanh((2.0 / torch.pi) ** 0.5 * (want + 0.044715 * want ** 3)))
+        close(o, want, dtype, f"rows {gr.begin}..{gr.end}")
+    assert bool((wide[:, :16] == 9.0).all()) and bool((wide[:, 48:] == 9.0).all())
+
+
+MIXER_GEOMS = [
+    dict(), dict(heads=4, kv_heads=2, dim=32, vdim=16, heads_2=2, dim_2=64, rot_dims=16, rot_dims_2=64),
+    dict(heads=3, kv_heads=1, dim=7, vdim=5, heads_2=1, dim_2=9, rot_dims=6, rot_dims_2=2, rot_scaling=None),
+    dict(heads=2, kv_heads=2, heads_2=2, window=None, vdim=33),
+    dict(heads=32, kv_heads=1, dim=16, vdim=16, window=5, heads_2=16, dim_2=16, window_2=1, rot_dims_2=4),
+    dict(heads=1, kv_heads=1, heads_2=1, dim=4, vdim=1, dim_2=2, rot_dims=4, rot_dims_2=0, window=1, keep_first=0),
+]
+
+
+@pytest.mark.parametrize("mode", MODES)
+@pytest.mark.parametrize("layer", ["ad", "a-", "bd", "b-"])
+@pytest.mark.parametrize("k", range(len(MIXER_GEOMS)))
+def test_layer_alone(mode, layer, k):
+    """One layer: the residual after it is norm(embedding) + (mixer(norm1) +
+    ff(norm2)); read in portions so that later ones continue the cache."""
+    device, dtype = mode
+    _skip_if_wrong_device(device)
+    cfg = make_cfg(layer, **MIXER_GEOMS[k])
+    W = O.random_weights(cfg, seed=3 + k)
+    eng = build_engine(cfg, W, dtype)
+    toks = tokens_for(cfg, 33, k)
+    _, layers, noisy = oracle_runs(cfg, rounded(W, dtype), toks, dtype)
+    eng.model.trace_layers = []
+    parts = cut(toks, [17, 1, 2, 13])
+    replay(eng, [[("a", p, i == len(parts) - 1)] for i, p in enumerate(parts)])
+    got = torch.cat(eng.model.trace_layers, 0)
+    close_rows(got, layers[0], [ls[0] for _, ls in noisy], dtype, f"{layer} geometry {k}")
+
+
+@pytest.mark.parametrize("mode", MODES)
+@pytest.mark.parametrize("pattern,first", [("AdBdAd", 0), ("bdadBdadAd", 2), ("B-A-", 0), ("adBd", 1), ("adbd", None)])
+def test_value_mixing(mode, pattern, first):
+    """Later mixing layers take lambda of the FIRST mixing layer's values,
+    bias included, whichever kind and place that layer has; with lambda 1 they
+    take nothing else, and 0 or more than 1 are as good. What is cached is the
+    mixed value."""
+    device, dtype = mode
+    _skip_if_wrong_device(device)
+    cfg = make_cfg(pattern)
+    spec = safesun_spec_from_dict(cfg)
+    mixing = [i for i, L in enumerate(cfg["layers"]) if L["mixer"]["v_mix"]]
+    assert [L.mixer.v_first_from for L in spec.layers] == [
+        first if i in mixing[1:] else None for i in range(len(spec.layers))]
+    for lam in (1.0, 0.0, 1.7):
+        W = O.random_weights(cfg, seed=6)
+        for i in mixing:
+            W[f"l{i}.mix.vmix"] = torch.tensor(lam)
+        eng = build_engine(cfg, W, dtype)
+        toks = tokens_for(cfg, 24, 3)
+        model_close(serve(eng, toks, [10, 1, 2, 11]), cfg, W, toks, dtype, f"lambda {lam}")
+        if lam == 1.0 and len(mixing) > 1:
+            for i in mixing[1:]:
+                assert torch.equal(eng.kv.layers[i][1], eng.kv.layers[first][1])
+
+
+# --------------------------------------------------------------------------
+# whole models
+
+
+@pytest.fixture(scope="module", params=["odd", "x16"])
+def model_case(request):
+    cfg = make_cfg() if request.param == "odd" else x16_cfg()
+    return cfg, O.random_weights(cfg, seed=1)
+
+
+@pytest.mark.parametrize("mode", MODES)
+def test_layers_and_logits_whole_prompt(mode, model_case):
+    device, dtype = mode
+    _skip_if_wrong_device(device)
+    cfg, W = model_case
+    eng = build_engine(cfg, W, dtype)
+    toks = tokens_for(cfg, 45, 2)
+    want, layers, noisy = oracle_runs(cfg, rounded(W, dtype), toks, dtype)
+    plain = serve(eng, toks, [45])
+    eng.model.trace_layers = []
+    got = serve(eng, toks, [45])
+    assert len(eng.model.trace_layers) == len(layers)
+    for i, x in enumerate(eng.model.trace_layers):
+        close_rows(x, layers[i], [ls[i] for _, ls in noisy], dtype, f"residual after layer {i}")
+    close_rows(got, want, [lg for lg, _ in noisy], dtype, "logits")
+    close_rows(plain, want, [lg for lg, _ in noisy], dtype, "logits without the layer trace")
+
+
+@pytest.mark.parametrize("mode", MODES)
+def test_first_tokens(mode, model_case):
+    device, dtype = mode
+    _skip_if_wrong_device(device)
+    cfg, W = model_case
+    eng = build_engine(cfg, W, dtype)
+    for n in (1, 2, 3, 6):
+        toks = tokens_for(cfg, n, 10 + n)
+        model_close(serve(eng, toks, [n]), cfg, W, toks, dtype, f"{n} tokens at once")
+        model_close(serve(eng, toks, [1]), cfg, W, toks, dtype, f"{n} tokens one by one")
+
+
+@pytest.mark.parametrize("mode", MODES)
+@pytest.mark.parametrize("sizes", [[1], [2], [3, 2], [7, 1, 2], [8], [16, 5], [9, 1, 1, 30], [21, 22]])
+def test_portions_and_decode(mode, model_case, sizes):
+    """Any cut of the prompt, token-by-token decoding included, gives the
+    logits of the whole prompt at once."""
+    device, dtype = mode
+    _skip_if_wrong_device(device)
+    cfg, W = model_case
+    eng = build_engine(cfg, W, dtype)
+    toks = tokens_for(cfg, 61, 3)
+    model_close(serve(eng, toks, sizes), cfg, W, toks, dtype, f"portions {sizes}")
+    assert eng.kv.num_free() == eng.kv.num_blocks and eng.state_pool.num_free() == 4
+
+
+@pytest.mark.parametrize("mode", MODES)
+def test_unequal_batch_equals_alone(mode, model_case):
+    """Four unequal requests share steps (portions beside single tokens, one
+    sitting out now and then); each equals itself alone."""
+    device, dtype = mode
+    _skip_if_wrong_device(device)
+    cfg, W = model_case
+    eng = build_engine(cfg, W, dtype)
+    reqs = {"a": tokens_for(cfg, 53, 4), "b": tokens_for(cfg, 9, 5), "c": tokens_for(cfg, 1, 7),
+            "d": tokens_for(cfg, 30, 7)}
+    plan = {"a": cut(reqs["a"], [11, 2, 1, 1, 19]), "b": cut(reqs["b"], [1]),
+            "c": [reqs["c"]], "d": cut(reqs["d"], [2, 13, 1])}
+    schedule, k = [], 0
+    while any(plan.values()):
+        step = []
+        for i in sorted(plan):
+            if plan[i] and not (i == "a" and k % 4 == 3):
+                p = plan[i].pop(0)
+                step.append((i, p, not plan[i]))
+        schedule.append(step)
+        k += 1
+    got = replay(eng, schedule)
+    for i, toks in reqs.items():
+        model_close(got[i], cfg, W, toks, dtype, f"request {i} in a mixed batch")
+
+
+@pytest.mark.parametrize("mode", MODES)
+def test_pages_and_slots_used_again(mode, model_case):
+    """A pool of 6 pages and 2 slots serves 7 requests in turn; freed pages
+    come back in another order and hold stale keys and values (also of the
+    layer whose values the others mix in)."""
+    device, dtype = mode
+    _skip_if_wrong_device(device)
+    cfg, W = model_case
+    eng = build_engine(cfg, W, dtype, blocks=6, block_size=8, slots=2)
+    lens = [20, 17, 25, 3, 24, 9, 22]
+    reqs = {"r%d" % k: tokens_for(cfg, n, 20 + k) for k, n in enumerate(lens)}
+    rp = TraceReplayer(eng)
+    names = list(reqs)
+    live, nxt, got = {}, 0, {i: [] for i in reqs}
+    while nxt < len(names) or live:
+        while nxt < len(names) and len(live) < 2:
+            need = sum((len(reqs[i]) + 7) // 8 for i in live) + (len(reqs[names[nxt]]) + 7) // 8
+            if need > 6:
+                break
+            live[names[nxt]] = cut(reqs[names[nxt]], [5, 1, 2, 7])
+            nxt += 1
+        entries, end = [], []
+        for i in list(live):
+            p = live[i].pop(0)
+            entries.append({"id": i, "tokens": p, "want": list(range(len(p)))})
+            if not live[i]:
+                end.append(i)
+                del live[i]
+        out = rp.step(entries, end)
+        off = 0
+        for e in entries:
+            got[e["id"]].append(out[off:off + len(e["tokens"])])
+            off += len(e["tokens"])
+    for i, toks in reqs.items():
+        model_close(torch.cat(got[i], 0), cfg, W, toks, dtype, f"{i} on reused pages")
+    assert eng.kv.num_free() == 6 and eng.state_pool.num_free() == 2
+
+
+@pytest.mark.parametrize("mode", MODES)
+def test_long_decode(mode):
+    """A short prompt, then 150 tokens one by one: the windows pass over
+    decoded tokens while the first ones stay in sight. Scores are sharp, so a
+    key too many or too few shows."""
+    device, dtype = mode
+    _skip_if_wrong_device(device)
+    cfg = make_cfg("AdBdAd", scale=0.8, scale_2=3.0)
+    W = O.random_weights(cfg, seed=8)
+    eng = build_engine(cfg, W, dtype)
+    toks = tokens_for(cfg, 170, 9)
+    parts = [toks[:20]] + [[t] for t in toks[20:]]
+    got = replay(eng, [[("a", p, k == len(parts) - 1)] for k, p in enumerate(parts)])["a"]
+    model_close(got, cfg, W, toks, dtype, "long decode")
+
+
+@pytest.mark.parametrize("mode", MODES)
+@pytest.mark.parametrize("keep", [4, 67])
+def test_long_portion(mode, keep):
+    """A portion longer than several key tiles, beside short ones, then
+    continued; kept tokens within one key tile and beyond it."""
+    device, dtype = mode
+    _skip_if_wrong_device(device)
+    cfg = x16_cfg("AdBd", window=100, window_2=70, keep_first=keep, keep_first_2=keep + 1, scale_2=2.0)
+    W = O.random_weights(cfg, seed=18)
+    eng = build_engine(cfg, W, dtype, blocks=128)
+    toks = tokens_for(cfg, 330, 9)
+    model_close(serve(eng, toks, [257, 1, 70, 2]), cfg, W, toks, dtype, "long portion")
+
+
+@pytest.mark.parametrize("mode", MODES)
+@pytest.mark.parametrize("kind", ["A", "B"])
+@pytest.mark.parametrize("where", ["kept", "first-not-kept", "in-window", "out-of-window"])
+def test_a_token_far_back_shows_in_the_logits(mode, kind, where):
+    """A one-layer model whose keys point one way for one marked token only,
+    the way every query points: changing the token's value changes the last
+    logits if the mask says so, and does not otherwise."""
+    device, dtype = mode
+    _skip_if_wrong_device(device)
+    n, win, keep = 60, 21, 4
+    at = {"kept": keep - 1, "first-not-kept": keep, "in-window": n - win, "out-of-window": n - win - 1}[where]
+    cfg = make_cfg(kind.lower() + "-", heads=2, heads_2=2, kv_heads=1, dim=12, dim_2=12, window=win, window_2=win,
+                   keep_first=keep, keep_first_2=keep, rot_dims=4, rot_dims_2=4, scale=3.0, scale_2=3.0)
+    W = O.random_weights(cfg, seed=13)
+    p = "l0.mix."
+    W["embed"] *= 0.2
+    W["embed"][:, 0] = 1.0                       # all tokens: channel 0
+    W["embed"][:, 1] = 0.0
+    W["embed"][95:97, 1] = 4.0                   # the two marked tokens: channel 1
+    for nm in ("q", "k"):
+        W[p + nm] *= 0.02
+        if kind == "B":
+            W[p + nm + ".b"] *= 0.0
+    W[p + "q"][11, 0] = W[p + "q"][23, 0] = 5.0    # an unrotated channel
+    W[p + "k"][11, 1], W[p + "k"][11, 0] = 5.0, -2.0
+    toks = [t % 90 for t in tokens_for(cfg, n, 5)]
+    outs = []
+    for mark in (95, 96):
+        toks[at] = mark
+        eng = build_engine(cfg, W, dtype)
+        for sizes in ([n], [n - 1, 1]):
+            got = serve(eng, toks, sizes)
+            model_close(got, cfg, W, toks, dtype, f"{where}, portions {sizes}")
+        outs.append(got[-1].double().cpu())
+    moved = (outs[0] - outs[1]).abs().max() / outs[0].abs().max()
+    assert (moved > 0.05) if where in ("kept", "in-window") else (moved < 1e-6), (where, moved)
+
+
+VARIANTS = {
+    # values that are often equal or 1, made different or extreme
+    "one-head": dict(heads=1, kv_heads=1, heads_2=1),
+    "heads-equal-kv-heads": dict(heads=3, kv_heads=3, heads_2=3),
+    "one-kv-head": dict(heads=5, kv_heads=1, heads_2=2),
+    "window-1": dict(window=1, window_2=2),
+    "window-8": dict(window=8, window_2=16),
+    "no-window": dict(window=None, window_2=0),
+    "window-in-one-kind": dict(window=None, window_2=9),
+    "keep-none": dict(keep_first=0, keep_first_2=0),
+    "keep-one": dict(keep_first=1, keep_first_2=1, window=3, window_2=4),
+    "keep-more-than-window": dict(keep_first=11, keep_first_2=17, window=5, window_2=6),
+    "keep-all": dict(keep_first=99, keep_first_2=99, window=5, window_2=6),
+    "unit-constants": dict(scale=1.0, scale_2=1.0),
+    "sharp": dict(scale=2.0, scale_2=4.0),
+    "flat": dict(scale=0.01, scale_2=0.01),
+    "rotate-all": dict(rot_dims=12, rot_dims_2=14),
+    "rotate-little": dict(rot_dims=2, rot_dims_2=2),
+    "rotate-none": dict(rot_dims=0, rot_dims_2=0, rot_scaling=None),
+    "no-scaling": dict(rot_scaling=None),
+    "strong-scaling": dict(rot_scaling=dict(factor=50.0, fast=2.0, slow=0.2, original=40)),
+    "scaling-from-the-first-pair": dict(rot_scaling=dict(factor=8.0, fast=300.0, slow=100.0, original=40)),
+    "wide-values": dict(vdim=70),
+    "wide-keys": dict(dim=68, dim_2=36, vdim=4, rot_dims=36),
+    "big-eps": dict(eps=0.3),
+    "odd-width": dict(width=39),
+    "tiny-ff": dict(ff=3),
+}
+
+
+@pytest.mark.parametrize("mode", MODES)
+@pytest.mark.parametrize("variant", sorted(VARIANTS))
+def test_other_sizes(mode, variant):
+    device, dtype = mode
+    _skip_if_wrong_device(device)
+    cfg = make_cfg("BdadA-Bd", **VARIANTS[variant])
+    W = O.random_weights(cfg, seed=11)
+    eng = build_engine(cfg, W, dtype)
+    toks = tokens_for(cfg, 40, 12)
+    model_close(serve(eng, toks, [13, 2, 1, 1, 9]), cfg, W, toks, dtype, variant)
+
+
+def test_scaling_in_the_second_kind():
+    """The rotation of either kind takes a scaling when the config gives one;
+    the magnitude then cancels in the unit norm except for passing channels."""
+    cfg = make_cfg("BdAd", rot_dims_2=6)
+    for L in cfg["layers"]:
+        L["mixer"]["rot"]["scaling"] = dict(YARN, factor=9.0)
+    W = O.random_weights(cfg, seed=17)
+    eng = build_engine(cfg, W)
+    if eng.device == "cuda":
+        pytest.skip("covered on CPU runs")
+    toks = tokens_for(cfg, 40, 12)
+    model_close(serve(eng, toks, [23, 17]), cfg, W, toks, "fp32", "scaled second kind")
+
+
+@pytest.mark.parametrize("mode", MODES)
+def test_prefix_pages_are_reused(mode, model_case):
+    """No layer carries state, so a second request that shares a prefix starts
+    from its pages; the values that later layers mix in are those of the new
+    tokens only."""
+    device, dtype = mode
+    _skip_if_wrong_device(device)
+    cfg, W = model_case
+    eng = build_engine(cfg, W, dtype)
+    assert eng.kv.prefix_caching and not any(eng.state_pool.tensors)
+    a = tokens_for(cfg, 37, 71)
+    b = a[:29] + tokens_for(cfg, 12, 72)
+    params = SamplingParams(max_new_tokens=6, stop_on_eos=False)
+    eng.generate(a, params)
+    before = eng.kv.stats["reused_blocks"]
+    out, _ = eng.generate(b, params)
+    assert eng.kv.stats["reused_blocks"] - before == 3
+    if dtype == "fp32":
+        assert out == O.greedy(cfg, W, b, 6)
+    else:
+        fresh = build_engine(cfg, W, dtype)
+        model_close(serve(fresh, b, [24, 17]), cfg, W, b, dtype, "after a prefix of three pages")
+
+
+def test_config_reader_takes_every_constant():
+    """Every size and constant of config.json lands in the spec."""
+    cfg = make_cfg("adBdA-")
+    spec = safesun_spec_from_dict(cfg)
+    assert (spec.layer_style, spec.embed_norm, spec.tied_head, spec.norm_eps, spec.vocab_size,
+            spec.hidden_size) == ("parallel_rms", True, True, 1e-5, 97, 42)
+    a, b = spec.layers[0].mixer, spec.layers[1].mixer
+    assert (a.kind, a.heads, a.kv_heads, a.dim, a.vdim, a.window, a.keep_first, a.scale) == (
+        "gated_rotary", 6, 2, 12, 10, 21, 3, 0.4)
+    assert (a.rot_dims, a.rot_base, a.rot_scaling, a.rot_layout) == (8, 3000.0, YARN, "half")
+    assert (a.qk_norm, a.qkv_bias, a.plus_one, a.v_mix, a.gate) == ("weighted", False, False, False, "channel")
+    assert (b.heads, b.dim, b.window, b.keep_first, b.scale, b.rot_dims, b.rot_base, b.rot_scaling) == (
+        4, 14, 13, 5, 1.1, 14, 700.0, None)
+    assert (b.qk_norm, b.qkv_bias, b.plus_one, b.v_mix) == ("unit_rotated", True, True, True)
+    assert [L.mixer.v_first_from for L in spec.layers] == [None, None, 1]
+    assert a.has_kv and not a.has_state
+    assert (spec.layers[0].mlp_kind, spec.layers[0].mlp_ff, spec.layers[0].mlp_act) == ("dense", 52, "silu")
+    assert spec.layers[2].mlp_kind is None
+    bare = copy.deepcopy(cfg)
+    for key in ("mask", "rot", "scale", "v_mix"):
+        bare["layers"][0]["mixer"].pop(key, None)
+    a = safesun_spec_from_dict(bare).layers[0].mixer
+    assert (a.window, a.keep_first, a.rot_dims, a.scale, a.v_mix) == (None, 0, 0, None, False)
+    for edit in (lambda c: c["layers"][0].update(type="convolution"),
+                 lambda c: c["layers"][0]["mlp"].update(kind="moe"),
+                 lambda c: c["layers"][0]["mixer"]["rot"].update(dims=5),
+                 lambda c: c["layers"][0]["mixer"]["rot"].update(dims=20),
+                 lambda c: c["layers"][2]["mixer"].update(vdim=4),
+                 lambda c: c["layers"][1]["mixer"].update(kv_heads=3)):
+        bad = copy.deepcopy(cfg)
+        edit(bad)
+        with pytest.raises(ValueError):
+            safesun_spec_from_dict(bad)
+
+
+def test_checkpoint_folder_roundtrip(tmp_path):
+    """A folder with config.json and model.safetensors (bfloat16) is found by
+    its architecture name and serves the oracle's logits."""
+    from safetensors.torch import save_file
+
+    cfg = make_cfg("adBdA-", width=32)
+    W = {k: v.to(torch.bfloat16) for k, v in O.random_weights(cfg, seed=2).items()}
+    (tmp_path / "config.json").write_text(json.dumps(cfg))
+    save_file({k: v.contiguous() for k, v in W.items()}, str(tmp_path / "model.safetensors"))
+    if torch.cuda.is_available():
+        pytest.skip("covered on CPU runs")
+    eng = LLMEngine({"model": str(tmp_path), "dtype": "fp32", "kv_num_blocks": 16, "kv_block_size": 8,
+                     "max_batch_size": 2, "state_slots": 2, "tokenizer_check": False})
+    assert eng.spec.architecture == "Safesun" and eng.model.lm_head is eng.model.embed
+    toks = tokens_for(cfg, 20, 1)
+    close(serve(eng, toks, [20]), O.forward(cfg, {k: v.float() for k, v in W.items()}, toks), "fp32", "folder")
+    missing = {k: v for k, v in W.items() if k != "l1.mix.k.b"}
+    with pytest.raises(KeyError):
+        eng.model.load_named_tensors(missing)
+
+
+# --------------------------------------------------------------------------
+# generation through the engine's own entry point and scheduler
+
+
+@pytest.mark.parametrize("mode", MODES[:2])
+def test_greedy_generation_matches_oracle(mode, model_case):
+    device, dtype = mode
+    _skip_if_wrong_device(device)
+    cfg, W = model_case
+    eng = build_engine(cfg, W, dtype, max_prefill_chunk=16)     # prompt read in portions
+    prompt = tokens_for(cfg, 37, 30)
+    out, reason = eng.generate(prompt, SamplingParams(max_new_tokens=24, stop_on_eos=False))
+    assert reason == "length"
+    assert out == O.greedy(cfg, W, prompt, 24)
+
+
+@pytest.mark.parametrize("mode", MODES)
+def test_scheduler_batches_equal_solo(mode, model_case):
+    """Five requests through add_request/step with two slots: admission waits
+    for a free slot, portions and decodes share forwards, and every output
+    equals the request generated alone."""
+    device, dtype = mode
+    _skip_if_wrong_device(device)
+    cfg, W = model_case
+    prompts = [tokens_for(cfg, n, 40 + n) for n in (5, 33, 1, 18, 9)]
+    params = SamplingParams(max_new_tokens=10, stop_on_eos=False)
+    solo = []
+    eng = build_engine(cfg, W, dtype, max_prefill_chunk=12)
+    for p in prompts:
+        solo.append(eng.generate(p, params)[0])
+    eng2 = build_engine(cfg, W, dtype, slots=2, max_prefill_chunk=12)
+    rids = [eng2.add_request(p, params) for p in prompts]
+    for _ in range(400):
+        if all(eng2.requests[r].finished for r in rids):
+            break
+        eng2.step()
+    if dtype == "fp32":
+        assert [eng2.requests[r].output_ids for r in rids] == solo
+    else:
+        assert all(len(eng2.requests[r].output_ids) == 10 for r in rids)
+    assert eng2.state_pool.num_free() == 2 and eng2.kv.num_free() == eng2.kv.num_blocks
+
+
+@gpu
+@pytest.mark.parametrize("dtype", ["fp32", "bf16"])
+@pytest.mark.parametrize("requests", [2, 3])
+def test_decode_graph_equals_eager(dtype, requests, model_case):
+    """Decode-only steps replay a captured graph per batch bucket (three
+    requests pad a bucket of four); several replays, with eager portions
+    between them, equal the eager engine."""
+    cfg, W = model_case
+    reqs = {i: tokens_for(cfg, 40, 50 + k) for k, i in enumerate("abc"[:requests])}
+    at = {i: n for i, n in zip(reqs, (20, 9, 15))}
+    sched = [[(i, reqs[i][: at[i]], False) for i in reqs]]
+    for _ in range(10):
+        sched.append([(i, [reqs[i][at[i]]], False) for i in reqs])
+        at = {i: n + 1 for i, n in at.items()}
+    sched.append([("x", reqs["a"][:15], True), ("b", [reqs["b"][at["b"]]], False)])
+    at["b"] += 1
+    for _ in range(6):
+        sched.append([(i, [reqs[i][at[i]]], False) for i in reqs])
+        at = {i: n + 1 for i, n in at.items()}
+    outs = []
+    for graph in (False, True):
+        eng = build_engine(cfg, W, dtype, use_hipgraph=graph)
+        outs.append(replay(eng, copy.deepcopy(sched)))
+        if graph:
+            assert any(e["graph"] is not None for e in eng._graphs.values())
+    for i in outs[0]:
+        if requests == 2:
+            # a captured step splits the keys for the longest context of the pool
+            close(outs[1][i], outs[0][i], "fp32" if dtype == "fp32" else "bf16", f"graph replay of {i}")
+        else:
+            # the padded bucket runs its products with another row count
+            close(outs[1][i], outs[0][i], dtype, f"padded graph replay of {i}", loose=3.0)
+    for i, toks in reqs.items():
+        model_close(outs[1][i], cfg, W, toks[: at[i]], dtype, f"graphed {i}")
+
+
+@gpu
+def test_wide_layers_take_the_decode_kernels():
+    """Layer widths of the decode kernels' matrix-core form (K a multiple of
+    1024), output products deep enough to be cut: batches of 1, 2 and 5
+    decoded tokens against the oracle."""
+    cfg = make_cfg("AdBdAd", width=1024, heads=8, kv_heads=2, dim=64, vdim=128, heads_2=8, dim_2=64, rot_dims=64,
+                   rot_dims_2=32, ff=4096, scale=0.125, scale_2=0.5)
+    W = O.random_weights(cfg, seed=31)
+    eng = build_engine(cfg, W, "bf16", slots=8)
+    for n in (1, 2, 5):
+        reqs = {"q%d" % k: tokens_for(cfg, 24, 60 + k) for k in range(n)}
+        sched = [[(i, t[:20], False) for i, t in reqs.items()]]
+        for k in range(20, 24):
+            sched.append([(i, [t[k]], k == 23) for i, t in reqs.items()])
+        got = replay(eng, sched)
+        for i, t in reqs.items():
+            model_close(got[i], cfg, W, t, "bf16", f"{i} of {n}")
+
+
+def test_named_sizes_build():
+    """The registry's Safesun sizes parse; the CPU-test size serves tokens."""
+    for name in ("safesun-tiny", "safesun-micro", "safesun-4l2k", "safesun-4l4k"):
+        spec = get_model_spec(name)
+        assert spec.architecture == "Safesun" and spec.layer_style == "parallel_rms"
+    if torch.cuda.is_available():
+        pytest.skip("generation on the CPU path is covered on CPU runs")
+    eng = LLMEngine({"model": "safesun-tiny", "dtype": "fp32", "kv_num_blocks": 32,
+                     "kv_block_size": 8, "max_batch_size": 2, "state_slots": 2,
+                     "tokenizer_check": False})
+    out, reason = eng.generate([5, 6, 7, 8, 9], SamplingParams(max_new_tokens=6, stop_on_eos=False))
+    assert len(out) == 6 and reason == "length"

@@ -1387,6 +1387,8 @@ class HybridForCausalLM(nn.Module):
         )
         self.embed_norm_w = None
         if spec.embed_norm:
+            if spec.sinusoid or spec.embed_scale != 1.0:
+                raise ValueError("a normed embedding takes no scale and no position vector")
             self.embed_norm_w = _param(0.05 * _rand(gen, 1, C))
         if self.rms:
             self.final_norm_w = _param(torch.zeros(1, C, device=device))
@@ -1431,10 +1433,11 @@ class HybridForCausalLM(nn.Module):
     def forward(self, fb: ForwardBatch, kv_caches, state=None) -> torch.Tensor:
         sb = fb.seq_batch
         assert sb is not None and state is not None, "hybrid models run flat multi-sequence steps"
-        x = mx.embed_rows(self.embed, fb.input_ids, self.spec.embed_scale, self.pos_freq, sb)
         if self.embed_norm_w is not None:
-            x = mx.add_rms_norm(x, self.embed_norm_w, self.spec.norm_eps, torch.float32,
-                                offset=1.0)[0]
+            x = mx.embed_norm_rows(self.embed, fb.input_ids, self.embed_norm_w,
+                                   self.spec.norm_eps, offset=1.0)
+        else:
+            x = mx.embed_rows(self.embed, fb.input_ids, self.spec.embed_scale, self.pos_freq, sb)
         if self.parallel:
             e0 = x.clone() if self.loop_entries else None
             y = bias = None

@@ -926,17 +926,18 @@ __global__ __launch_bounds__(256) void attn_bias_mfma_kernel(
     }
 }
 
-// merge key-split partials: one wave per (token, head); lanes first take
-// one split each for the statistics, then one value channel each
+// merge key-split partials: one block per (token, head). Every wave first
+// takes the statistics of all splits, a lane each; then wave w adds up the
+// splits w, w + 4, ..., a lane per value channel, and the waves' sums meet in LDS
 template <typename TC>
-__global__ __launch_bounds__(64) void attn_combine_kernel(
+__global__ __launch_bounds__(256) void attn_combine_kernel(
     const float* __restrict__ part_o, const float* __restrict__ part_ml,
     const TC* __restrict__ gate, int64_t gs, const float* __restrict__ sinks,
     TC* __restrict__ out, int H, int Dv, int nsplit, int64_t os, float oscale, int gch) {
-    __shared__ float wsh[64];
+    __shared__ float sums[4][64 * ATT_MAXV];
     const int64_t row = blockIdx.x;  // tok * H + h
     const int tok = (int)(row / H), h = (int)(row % H);
-    const int lane = threadIdx.x;
+    const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
     float mx = -INFINITY, lsum = 0.0f;
     for (int s0 = 0; s0 < nsplit; s0 += 64) {          // running merge over groups of 64 splits
         const int s = s0 + lane;
@@ -948,36 +949,30 @@ __global__ __launch_bounds__(64) void attn_combine_kernel(
         mx = gmx;
     }
     if (sinks) lsum += expf(sinks[h] - mx);
-    const float gt = (gate && !gch ? sigmoidf_(ldf(gate, (int64_t)tok * gs + h)) : 1.0f) * oscale / lsum;
     float acc[ATT_MAXV];
 #pragma unroll
     for (int c = 0; c < ATT_MAXV; ++c) acc[c] = 0.0f;
-    for (int s0 = 0; s0 < nsplit; s0 += 64) {
-        const int s = s0 + lane;
-        const float ms = s < nsplit ? part_ml[(row * nsplit + s) * 2] : -INFINITY;
-        __syncthreads();
-        wsh[lane] = (ms == -INFINITY) ? 0.0f : expf(ms - mx);
-        __syncthreads();
-        const int ns = min(64, nsplit - s0);
 #pragma unroll 4
-        for (int j = 0; j < ns; ++j) {
-            const float wj = wsh[j];
-            const float* po = part_o + (row * nsplit + s0 + j) * Dv;
+    for (int s = wave; s < nsplit; s += 4) {
+        const float ms = part_ml[(row * nsplit + s) * 2];
+        const float wj = (ms == -INFINITY) ? 0.0f : expf(ms - mx);
+        const float* po = part_o + (row * nsplit + s) * Dv;
 #pragma unroll
-            for (int c = 0; c < ATT_MAXV; ++c) {
-                const int ch = lane + 64 * c;
-                if (ch < Dv) acc[c] += po[ch] * wj;
-            }
+        for (int c = 0; c < ATT_MAXV; ++c) {
+            const int ch = lane + 64 * c;
+            if (ch < Dv) acc[c] += po[ch] * wj;
         }
     }
 #pragma unroll
-    for (int c = 0; c < ATT_MAXV; ++c) {
-        const int ch = lane + 64 * c;
-        if (ch >= Dv) continue;
-        float v = acc[c] * gt;
-        if (gate && gch) v *= sigmoidf_(ldf(gate, (int64_t)tok * gs + h * Dv + ch));
-        stf(out, (int64_t)tok * os + h * Dv + ch, v);
-    }
+    for (int c = 0; c < ATT_MAXV; ++c) sums[wave][lane + 64 * c] = acc[c];
+    __syncthreads();
+    const int ch = threadIdx.x;                        // Dv <= 64 * ATT_MAXV = 256
+    if (ch >= Dv) return;
+    float v = (sums[0][ch] + sums[1][ch]) + (sums[2][ch] + sums[3][ch]);
+    // in the order of the unsplit kernels: one split that saw every key gives their result
+    v *= (gate && !gch ? sigmoidf_(ldf(gate, (int64_t)tok * gs + h)) : 1.0f) * oscale / lsum;
+    if (gate && gch) v *= sigmoidf_(ldf(gate, (int64_t)tok * gs + h * Dv + ch));
+    stf(out, (int64_t)tok * os + h * Dv + ch, v);
 }
 
 // ---------------------------------------------------------------------------
@@ -1686,11 +1681,11 @@ extern "C" int oa_attn_bias_paged(void* stream, const void* q, const void* gate,
     }
     if (nsplit > 1) {
         if (dt == 1)
-            hipLaunchKernelGGL((attn_combine_kernel<float>), dim3((unsigned)((int64_t)T * H)), dim3(64), 0, s,
+            hipLaunchKernelGGL((attn_combine_kernel<float>), dim3((unsigned)((int64_t)T * H)), dim3(256), 0, s,
                                (const float*)part_o, (const float*)part_ml, (const float*)gate, gs,
                                (const float*)sinks, (float*)out, H, Dv, nsplit, os, oscale, gch);
         else
-            hipLaunchKernelGGL((attn_combine_kernel<bf16s>), dim3((unsigned)((int64_t)T * H)), dim3(64), 0, s,
+            hipLaunchKernelGGL((attn_combine_kernel<bf16s>), dim3((unsigned)((int64_t)T * H)), dim3(256), 0, s,
                                (const float*)part_o, (const float*)part_ml, (const bf16s*)gate, gs,
                                (const float*)sinks, (bf16s*)out, H, Dv, nsplit, os, oscale, gch);
         HIP_CHECK_LAUNCH();

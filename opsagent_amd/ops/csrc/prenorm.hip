@@ -186,51 +186,65 @@ extern "C" int oa_add_layer_norm(void* stream, void* residual, const void* y, in
 //   r = residual + y          (y optional: ny partial planes yp elements apart
 //                              that add up)
 //   residual = r              (if anything was added)
+//   ids given: r = y[ids[t]]  (y is a table; there is no residual)
 //   out_p = r / sqrt(mean(r^2) + eps) * (offset + w_p),  p < P
 // P norms of the same row with weights of their own (w [P, C], float32) go to
-// P planes of out, plane elements apart. One block per token; the first
-// 256 * LN_NR channels stay in registers, wider rows re-read the (just
-// written) residual for the rest.
-template <typename TY, typename TO, bool VEC>
-__global__ __launch_bounds__(256) void add_rms_norm_kernel(
+// P planes of out, plane elements apart. One block of NT threads per token (1024
+// where there are few tokens: a row's latency is then one or two loads); the
+// first 256 * LN_NR channels stay in registers, wider rows are read again for
+// the rest. Partial planes are loaded four at a time, then added in order.
+template <typename TY, typename TO, bool VEC, int NT>
+__global__ __launch_bounds__(NT) void add_rms_norm_kernel(
     float* __restrict__ residual, const TY* __restrict__ y, int64_t ys, int ny, int64_t yp,
-    const float* __restrict__ w, int P, float offset, TO* __restrict__ out, int64_t plane, int C,
-    float eps) {
+    const int64_t* __restrict__ ids, const float* __restrict__ w, int P, float offset,
+    TO* __restrict__ out, int64_t plane, int C, float eps) {
     __shared__ float red[16];
     constexpr int W = VEC ? 4 : 1;
-    constexpr int NS = LN_NR / W;
+    constexpr int NS = LN_NR * 256 / (W * NT);
     const int t = blockIdx.x, tid = threadIdx.x;
     float* r = residual + (int64_t)t * C;
+    const TY* yr = y + (ids ? ids[t] : (int64_t)t) * ys;
+    auto reload = [&](int c, float* x) {
+        if (ids) ldv<W>(yr, c, x);
+        else ldv<W>(r, c, x);
+    };
     auto load = [&](int c, float* x) {
-        ldv<W>(r, c, x);
-        if (!y) return;
-        for (int k = 0; k < ny; ++k) {
-            float a[W];
-            ldv<W>(y, k * yp + (int64_t)t * ys + c, a);
+        reload(c, x);
+        if (!y || ids) return;
+        for (int k = 0; k < ny; k += 4) {
+            float a[4][W];
 #pragma unroll
-            for (int e = 0; e < W; ++e) x[e] += a[e];
+            for (int q = 0; q < 4; ++q) {
+#pragma unroll
+                for (int e = 0; e < W; ++e) a[q][e] = 0.0f;
+                if (k + q < ny) ldv<W>(yr, (k + q) * yp + c, a[q]);
+            }
+#pragma unroll
+            for (int q = 0; q < 4; ++q)
+#pragma unroll
+                for (int e = 0; e < W; ++e) x[e] += a[q][e];
         }
         stv<W>(r, c, x);
     };
-    float vals[LN_NR];
+    float vals[NS * W];
     float ss = 0.0f;
 #pragma unroll
     for (int j = 0; j < NS; ++j) {
-        const int c = (tid + 256 * j) * W;
+        const int c = (tid + NT * j) * W;
 #pragma unroll
         for (int e = 0; e < W; ++e) vals[j * W + e] = 0.0f;
         if (c < C) load(c, vals + j * W);
 #pragma unroll
         for (int e = 0; e < W; ++e) ss += vals[j * W + e] * vals[j * W + e];
     }
-    for (int c = (tid + 256 * NS) * W; c < C; c += 256 * W) {
+    for (int c = (tid + NT * NS) * W; c < C; c += NT * W) {
         float x[W];
         load(c, x);
 #pragma unroll
         for (int e = 0; e < W; ++e) ss += x[e] * x[e];
     }
     if (!w) return;
-    const float rs = 1.0f / sqrtf(block_reduce_sum<4>(ss, red) / (float)C + eps);
+    const float rs = 1.0f / sqrtf(block_reduce_sum<NT / 64>(ss, red) / (float)C + eps);
     TO* o = out + (int64_t)t * C;
     auto emit = [&](int c, const float* x) {
         for (int p = 0; p < P; ++p) {
@@ -243,21 +257,23 @@ __global__ __launch_bounds__(256) void add_rms_norm_kernel(
     };
 #pragma unroll
     for (int j = 0; j < NS; ++j) {
-        const int c = (tid + 256 * j) * W;
+        const int c = (tid + NT * j) * W;
         if (c < C) emit(c, vals + j * W);
     }
-    for (int c = (tid + 256 * NS) * W; c < C; c += 256 * W) {
+    for (int c = (tid + NT * NS) * W; c < C; c += NT * W) {
         float x[W];
-        ldv<W>(r, c, x);
+        reload(c, x);
         emit(c, x);
     }
 }
 
 extern "C" int oa_add_rms_norm(void* stream, void* residual, const void* y, int64_t ys, int ny,
-                               int64_t yp, int y_dt, const void* w, int P, float offset, void* out,
-                               int64_t plane, int out_dt, int T, int C, float eps) {
+                               int64_t yp, int y_dt, const void* ids, const void* w, int P,
+                               float offset, void* out, int64_t plane, int out_dt, int T, int C,
+                               float eps) {
     if (T <= 0 || C <= 0) return 0;
-    if (!residual || (y && ny < 1) || (w && (!out || P < 1 || plane < (int64_t)T * C))) return -100;
+    if ((y && ny < 1) || (w && (!out || P < 1 || plane < (int64_t)T * C))) return -100;
+    if (ids ? (!y || !w || ny != 1) : !residual) return -101;
     if (!y && !w) return 0;
     if (!y) y_dt = out_dt;
     if (!w) out_dt = y_dt;
@@ -265,13 +281,16 @@ extern "C" int oa_add_rms_norm(void* stream, void* residual, const void* y, int6
     auto al = [](const void* p, int dt) { return !p || (uintptr_t)p % (dt == 1 ? 16 : 8) == 0; };
     const bool vec = C % 4 == 0 && ys % 4 == 0 && yp % 4 == 0 && plane % 4 == 0 && al(residual, 1) &&
                      al(w, 1) && al(y, y_dt) && al(out, out_dt);
-#define RN_LAUNCH(TY, TO, V)                                                                       \
-    hipLaunchKernelGGL((add_rms_norm_kernel<TY, TO, V>), dim3(T), dim3(256), 0, s, (float*)residual, \
-                       (const TY*)y, ys, ny, yp, (const float*)w, P, offset, (TO*)out, plane, C, eps)
-#define RN(TY, TO)                      \
-    do {                                \
-        if (vec) RN_LAUNCH(TY, TO, true); \
-        else RN_LAUNCH(TY, TO, false);  \
+    const bool wide = vec && T <= 256 && C > 1024;
+#define RN_LAUNCH(TY, TO, V, NT)                                                                   \
+    hipLaunchKernelGGL((add_rms_norm_kernel<TY, TO, V, NT>), dim3(T), dim3(NT), 0, s,              \
+                       (float*)residual, (const TY*)y, ys, ny, yp, (const int64_t*)ids,            \
+                       (const float*)w, P, offset, (TO*)out, plane, C, eps)
+#define RN(TY, TO)                                \
+    do {                                          \
+        if (wide) RN_LAUNCH(TY, TO, true, 1024);  \
+        else if (vec) RN_LAUNCH(TY, TO, true, 256); \
+        else RN_LAUNCH(TY, TO, false, 256);       \
     } while (0)
     if (y_dt == 1 && out_dt == 1) RN(float, float);
     else if (y_dt == 1) RN(float, bf16s);

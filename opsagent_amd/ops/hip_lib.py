@@ -158,7 +158,7 @@ def _declare_mixers(lib: ctypes.CDLL) -> None:
         "oa_rope_rows": [p, p, i64, i, p, i, i, i, p, i, p, p, p, i, i],
         "oa_combine_norm_gate": [p, p, i64, i, p, i64, f, p, i64, i, p, i, i, i, i, i, f, f],
         "oa_act_pair_rows": [p, p, i64, p, i64, i64, i, i, i],
-        "oa_add_rms_norm": [p, p, p, i64, i, i64, i, p, i, f, p, i64, i, i, i, f],
+        "oa_add_rms_norm": [p, p, p, i64, i, i64, i, p, p, i, f, p, i64, i, i, i, f],
         "oa_act_rows": [p, p, i64, p, i64, i64, i, i, i],
         "oa_moe_pairs_up": [p, p, p, p, p, i, i, i, i, i, i, i],
     }

@@ -291,6 +291,10 @@ def attention_paged(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tenso
     nsplit = 1
     if ntiles * G < 256 and nkt >= 8:
         nsplit = int(min(nkt // 4, max(1, 512 // max(1, ntiles * G)), 64))
+        if sb.max_chunk == 1:
+            # a decode step's blocks are short: down to two tiles each while
+            # that leaves at most 16 partials to merge
+            nsplit = max(nsplit, int(min(nkt // 2, max(1, 256 // (ntiles * G)), 16)))
     # decode steps of many query heads per kv head run one block per 64 heads
     # (the heads share each staged tile): fewer blocks, so finer key splits
     if (sb.max_chunk == 1 and H // G >= 16 and dt == 0 and D % 16 == 0 and Dv % 16 == 0
@@ -712,8 +716,28 @@ def add_rms_norm(residual: torch.Tensor, w: Optional[torch.Tensor], eps: float, 
         assert y.shape[-2:] == (T, C)
     rc = lib.oa_add_rms_norm(
         hip.current_stream_ptr(), residual.data_ptr(), y.data_ptr() if y is not None else None,
-        rows, ny, yp, _dt(y) if y is not None else 1, w.data_ptr() if w is not None else None, P,
+        rows, ny, yp, _dt(y) if y is not None else 1, None, w.data_ptr() if w is not None else None, P,
         float(offset), out.data_ptr() if P else None, T * C, _dt(out) if P else 1, T, C, float(eps))
+    hip.check(rc, "oa_add_rms_norm")
+    return out
+
+
+def embed_norm_rows(table: torch.Tensor, ids: torch.Tensor, w: torch.Tensor, eps: float,
+                    offset: float = 0.0) -> torch.Tensor:
+    """RMS norm of table[ids] with weight offset + w (float32 [C]), as a float32
+    residual stream [T, C]."""
+    C = table.shape[1]
+    assert w.dtype == torch.float32 and w.numel() == C and w.is_contiguous()
+    if not table.is_cuda:
+        return torch_ref.add_rms_norm(table[ids].float(), None, w.view(1, C), eps, torch.float32,
+                                      offset)[0]
+    lib, hip = _lib()
+    T = ids.shape[0]
+    assert ids.dtype == torch.int64 and ids.is_contiguous() and table.is_contiguous()
+    out = torch.empty(T, C, dtype=torch.float32, device=table.device)
+    rc = lib.oa_add_rms_norm(hip.current_stream_ptr(), None, table.data_ptr(), C, 1, 0, _dt(table),
+                             ids.data_ptr(), w.data_ptr(), 1, float(offset), out.data_ptr(), T * C,
+                             1, T, C, float(eps))
     hip.check(rc, "oa_add_rms_norm")
     return out
 
@@ -1163,13 +1187,17 @@ class RowGroup:
 
 # columns of K a block of the split product takes
 _SPLIT_UNIT = 4096
+# library products with a deeper K and at most so many rows run in two halves
+_HALVE_K, _HALVE_TOKENS = 16384, 2048
 
 
 def linear_partials(x: torch.Tensor, w: torch.Tensor) -> torch.Tensor:
     """x [T, K] @ w [N, K]^T for the deep output projection of a layer: [T, N]
-    in x's type, or, for decode batches that the matrix-core GEMV takes except
-    for their K, float32 partial sums [n, T, N] over pieces of K. The reader
-    (dyt_norm) adds them up."""
+    in x's type, or partial sums [n, T, N] over pieces of K that the reader
+    (dyt_norm, add_rms_norm) adds up: float32 for decode batches that the
+    matrix-core GEMV takes except for their K; in x's type, two halves of K,
+    for library products of up to _HALVE_TOKENS rows with a K above _HALVE_K,
+    where the library's choice for the whole K measured 1.4-1.9 times slower."""
     from opsagent_amd import ops
 
     T, K = x.shape
@@ -1184,6 +1212,13 @@ def linear_partials(x: torch.Tensor, w: torch.Tensor) -> torch.Tensor:
         hip.check(hip.get_lib().oa_gemv_split(hip.current_stream_ptr(), x.data_ptr(), w.data_ptr(),
                                               part.data_ptr(), T, N, K, _SPLIT_UNIT),
                   "oa_gemv_split")
+        return part
+    if (x.is_cuda and x.dtype == torch.bfloat16 and K > _HALVE_K and T <= _HALVE_TOKENS
+            and not ops._gemv_m_ok(T)):
+        half = (K // 2 + 63) // 64 * 64
+        part = torch.empty(2, T, N, dtype=x.dtype, device=x.device)
+        torch.mm(x[:, :half], w[:, :half].t(), out=part[0])
+        torch.mm(x[:, half:], w[:, half:].t(), out=part[1])
         return part
     return ops.linear(x, w)
 

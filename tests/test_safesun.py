@@ -436,6 +436,28 @@ def test_add_and_norms(mode, T, C, planes):
     out = mx.add_rms_norm(r, w.to(dev), 1e-6, torch.float32, offset=1.0)     # float32 rows in both modes
     assert out.dtype == torch.float32 and torch.equal(r.cpu(), res)
     close(out[0], O.norm(res.double(), w[0].double(), 1e-6), "fp32", "float32 norm")
+    table, ids = rn(6, C).to(dt), torch.tensor([5, 0, 3, 3, 1, 2, 4, 0, 5])[:T]
+    got = mx.embed_norm_rows(table.to(dev), ids.to(dev), w[0].to(dev), 0.1, offset=1.0)
+    assert got.dtype == torch.float32
+    close(got, O.norm(table[ids].double(), w[0].double(), 0.1), "fp32", "normed embedding rows")
+
+
+@gpu
+@pytest.mark.parametrize("T", [9, 40, 300])
+def test_deep_output_product_in_halves(T):
+    """Rows beyond the decode kernels with a deep K: two halves of K that the
+    norm kernel adds to the residual."""
+    g = torch.Generator().manual_seed(T)
+    K, N = 16384 + 80, 48
+    x = torch.randn(T, K, generator=g).to(torch.bfloat16)
+    w = (torch.randn(N, K, generator=g) * K ** -0.5).to(torch.bfloat16)
+    y = mx.linear_partials(x.cuda(), w.cuda())
+    assert y.shape == (2, T, N) and y.dtype == torch.bfloat16
+    want = x.double() @ w.double().T
+    close(y.double().sum(0), want, "bf16", "sum of the halves")
+    r = torch.zeros(T, N, device="cuda")
+    mx.add_rms_norm(r, None, 0.0, torch.bfloat16, y=y)
+    close(r, want, "bf16", "residual")
 
 
 @pytest.mark.parametrize("mode", MODES)

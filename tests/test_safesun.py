@@ -177,7 +177,7 @@ def serve(eng, toks, sizes):
 
 
 @pytest.mark.parametrize("dims,base,sc", [
-    (64, 20000.0, dict(factor=2.5, fast=32.0, slow=1.0, original=4096)),
+    (56, 15000.0, dict(factor=2.5, fast=32.0, slow=1.0, original=4096)),
     (16, 500.0, dict(factor=40.0, fast=4.0, slow=2.0, original=100)),
     (12, 10000.0, dict(factor=1.0, fast=32.0, slow=1.0, original=64)),
     (10, 10000.0, dict(factor=4.0, fast=1e9, slow=1e8, original=64)),       # both ends clamp to 0
@@ -302,13 +302,13 @@ def _attend_reference(dt, q, k, v, past, scale, mask, plus_one, gate=None):
     return o if gate is None else o * O.sigmoid(f(gate)).reshape(o.shape)
 
 
-WINDOW, KEEP = 72, 70      # neither a multiple of a page nor of a key tile
+WINDOW, KEEP = 77, 70      # neither a multiple of a page nor of a key tile
 
 
 @pytest.mark.parametrize("mode", MODES)
 @pytest.mark.parametrize("plus_one", [False, True])
 @pytest.mark.parametrize("keep", [5, KEEP])
-@pytest.mark.parametrize("target", [0, 1, 4, 5, 7, 8, 63, 64, 69, 70, 71, 150, -1, -8, -64, -71, -72, -73, -74, -80])
+@pytest.mark.parametrize("target", [0, 1, 4, 5, 7, 8, 63, 64, 69, 70, 71, 150, -1, -8, -64, -76, -77, -78, -79, -85])
 @pytest.mark.parametrize("n", [1, 9, 100])
 def test_one_key_stands_out(mode, plus_one, keep, target, n):
     """One key (a position, or so many before the end) has a large product
@@ -375,7 +375,7 @@ def test_extreme_scores_beside_the_one(mode, score):
 
 @pytest.mark.parametrize("mode", MODES)
 @pytest.mark.parametrize("H,G,D,Dv", [(6, 2, 12, 10), (4, 2, 32, 48), (3, 1, 7, 5), (32, 1, 16, 16), (5, 5, 64, 16),
-                                      (2, 2, 136, 8), (2, 1, 32, 272), (4, 1, 256, 128), (80, 2, 16, 32)])
+                                      (2, 2, 136, 8), (4, 2, 48, 80), (2, 1, 32, 272), (4, 1, 256, 128), (80, 2, 16, 32)])
 @pytest.mark.parametrize("size,keep", [(21, 3), (None, 0), (1, 1), (8, 64), (30, 0), (2, 200)])
 def test_attention_geometries(mode, H, G, D, Dv, size, keep):
     device, dtype = mode
